@@ -107,21 +107,42 @@ __global__ void __launch_bounds__(256) glu_clamp8_kernel(const TA* __restrict__ 
 // Router: one wave per token.  logits = Wr h in fp32; scores = sigmoid(logits)
 // (mode 0) or softmax (mode 1); the K largest (ties: lowest index), optionally
 // renormalised to sum 1 (divided by their sum + renorm_eps).  With `bias` [E] the
-// choice is made on score + bias while the weights stay the plain scores.  The weights are multiplied by
+// choice is made on score + bias while the weights stay the plain scores.  With NG > 0 the experts form NG equal
+// groups of neighbours: a group's score is the sum of its two largest choice scores, and only experts of the
+// `keep` best groups (ties: lowest index) can be chosen.  The weights are multiplied by
 // out_scale at the end.  wr may hold X more rows behind the E experts' (Et = E + X): their logits are not
 // routed but written as they are to extra[t][X] (per-token gates that read the same hidden row).
+// Expert e's score lives with lane e % 64, which forms, groups and marks it; a choice is a wave-wide argmax.
+__device__ __forceinline__ void wave_argmax(float& v, int& i) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ov = __shfl_xor(v, o, 64);
+    const int oi = __shfl_xor(i, o, 64);
+    if (ov > v || (ov == v && oi < i)) {
+      v = ov;
+      i = oi;
+    }
+  }
+}
+// LDS written by one lane is read by another of the same wave: no reordering across this point
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
 template <typename TA, typename TW>
 __global__ void __launch_bounds__(256) router_kernel(const TA* __restrict__ h, const TW* __restrict__ wr, int T, int W,
                                                      int Et, int K, int mode, int renorm, float* __restrict__ w_out,
                                                      int* __restrict__ id_out, const float* __restrict__ bias,
                                                      float renorm_eps, int X, float* __restrict__ extra,
-                                                     float out_scale) {
+                                                     float out_scale, int NG, int keep) {
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int t = blockIdx.x * 4 + wv;
   if (t >= T) return;
-  float* sc = sm + wv * 2 * Et;
+  float* sc = sm + wv * (2 * Et + NG);
   float* ch = sc + Et;   // choice scores
+  float* gs = ch + Et;   // group scores
   const int E = Et;      // rows whose logits are formed below; the routed ones are E - X
   if ((W & 7) == 0) {
     // 8 columns per lane and step, 16 experts at a time: the hidden row is read once per group
@@ -156,37 +177,77 @@ __global__ void __launch_bounds__(256) router_kernel(const TA* __restrict__ h, c
       if (lane == 0) sc[e] = a;
     }
   }
-  __builtin_amdgcn_wave_barrier();
-  if (lane == 0) {
+  wave_lds_fence();
+  {
     const int E = Et - X;
-    for (int x = 0; x < X; ++x) extra[(size_t)t * X + x] = sc[E + x];
+    for (int x = lane; x < X; x += 64) extra[(size_t)t * X + x] = sc[E + x];
     if (mode == 0) {
-      for (int e = 0; e < E; ++e) sc[e] = 1.f / (1.f + expf(-sc[e]));
+      for (int e = lane; e < E; e += 64) sc[e] = 1.f / (1.f + expf(-sc[e]));
     } else {
       float m = -INFINITY, s = 0.f;
-      for (int e = 0; e < E; ++e) m = fmaxf(m, sc[e]);
-      for (int e = 0; e < E; ++e) s += (sc[e] = expf(sc[e] - m));
-      for (int e = 0; e < E; ++e) sc[e] /= s;
+      for (int e = lane; e < E; e += 64) m = fmaxf(m, sc[e]);
+      m = wave_max(m);
+      for (int e = lane; e < E; e += 64) s += (sc[e] = expf(sc[e] - m));
+      s = wave_sum(s);
+      for (int e = lane; e < E; e += 64) sc[e] /= s;
     }
-    for (int e = 0; e < E; ++e) ch[e] = bias ? sc[e] + bias[e] : sc[e];
+    for (int e = lane; e < E; e += 64) ch[e] = bias ? sc[e] + bias[e] : sc[e];
+    wave_lds_fence();
+    if (NG > 0) {
+      const int n = E / NG;
+      for (int g = lane; g < NG; g += 64) {
+        float a = -INFINITY, b = -INFINITY;     // the two largest
+        for (int e = g * n; e < (g + 1) * n; ++e) {
+          const float v = ch[e];
+          if (v > a) {
+            b = a;
+            a = v;
+          } else {
+            b = fmaxf(b, v);
+          }
+        }
+        gs[g] = n > 1 ? a + b : a;
+      }
+      for (int k = 0; k < keep; ++k) {          // a kept group's score becomes -infinity
+        float bv = -INFINITY;
+        int bi = 1 << 30;
+        for (int g = lane; g < NG; g += 64)
+          if (gs[g] > bv) {
+            bv = gs[g];
+            bi = g;
+          }
+        wave_argmax(bv, bi);
+        if (bi < NG && (bi & 63) == lane) gs[bi] = -INFINITY;
+      }
+      wave_lds_fence();
+      for (int e = lane; e < E; e += 64)
+        if (gs[e / n] != -INFINITY) ch[e] = -INFINITY;
+    }
     float tot = 0.f;
     for (int k = 0; k < K; ++k) {
-      int bi = 0;
       float bv = -INFINITY;
-      for (int e = 0; e < E; ++e)
+      int bi = 1 << 30;
+      for (int e = lane; e < E; e += 64)
         if (ch[e] > bv) {
           bv = ch[e];
           bi = e;
         }
-      w_out[t * K + k] = sc[bi];
-      id_out[t * K + k] = bi;
-      tot += sc[bi];
-      ch[bi] = -INFINITY;
+      wave_argmax(bv, bi);
+      if (bi >= E) bi = k;                      // only where scores are not numbers: an index in range
+      const float v = sc[bi];
+      if ((bi & 63) == lane) ch[bi] = -INFINITY;
+      tot += v;
+      if (lane == 0) {
+        w_out[t * K + k] = v;
+        id_out[t * K + k] = bi;
+      }
     }
-    if (renorm)
-      for (int k = 0; k < K; ++k) w_out[t * K + k] /= (tot + renorm_eps);
-    if (out_scale != 1.f)
-      for (int k = 0; k < K; ++k) w_out[t * K + k] *= out_scale;
+    if (lane == 0) {
+      if (renorm)
+        for (int k = 0; k < K; ++k) w_out[t * K + k] /= (tot + renorm_eps);
+      if (out_scale != 1.f)
+        for (int k = 0; k < K; ++k) w_out[t * K + k] *= out_scale;
+    }
   }
 }
 
@@ -313,12 +374,14 @@ K8S_API int k8s_glu_clamp(const void* gu, void* out, int rows, int F, float alph
 
 K8S_API int k8s_router(const void* h, const void* wr, int T, int W, int E, int K, int mode, int renorm, float* w_out,
                        int* id_out, int dt, hipStream_t s, const float* bias, float renorm_eps, int X, float* extra,
-                       float out_scale) {
+                       float out_scale, int NG, int keep) {
   if (T <= 0) return 0;
-  if (K > E || E + X > 2048 || X < 0 || (X > 0 && !extra)) return (int)hipErrorInvalidValue;
-  K8S_DT(dt, hipLaunchKernelGGL((router_kernel<TA, TW>), dim3((T + 3) / 4), dim3(256), 8 * (E + X) * sizeof(float), s,
-                                 (const TA*)h, (const TW*)wr, T, W, E + X, K, mode, renorm, w_out, id_out, bias,
-                                 renorm_eps, X, extra, out_scale));
+  if (K < 1 || K > E || E + X > 1024 || X < 0 || (X > 0 && !extra) || NG < 0 ||
+      (NG > 0 && (E % NG || keep < 1 || keep > NG || keep * (E / NG) < K)))
+    return (int)hipErrorInvalidValue;
+  K8S_DT(dt, hipLaunchKernelGGL((router_kernel<TA, TW>), dim3((T + 3) / 4), dim3(256),
+                                 4 * (2 * (E + X) + NG) * sizeof(float), s, (const TA*)h, (const TW*)wr, T, W, E + X, K,
+                                 mode, renorm, w_out, id_out, bias, renorm_eps, X, extra, out_scale, NG, keep));
   return (int)hipGetLastError();
 }
 

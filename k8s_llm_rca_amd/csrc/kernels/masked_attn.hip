@@ -2,8 +2,9 @@
 // q and k.
 //
 // attn_prep:  rows of the joint projection (fp32: q [H][D] | k [G][D] | v [NV], row stride qs)
-//   + bias;  q, k rotated on their first `rot` entries per head (entry i with i + rot / 2, angle
-//   pos * base^(-2 i / rot), formed in double);  norm 1: q, k divided by the head's root mean square (eps inside
+//   + bias;  q, k rotated on their first `rot` entries per head (entry i with i + rot / 2, or with rot_pairs
+//   entry 2i with 2i + 1; angle pos * f_i with f_i = base^(-2 i / rot) or from a table of doubles, the product
+//   formed in double; cos and sin times rot_amp);  norm 1: q, k divided by the head's root mean square (eps inside
 //   the root) behind the rotation and multiplied by a weight [D] where given;  norm 2: q and k each divided by
 //   the root mean square of the WHOLE projection (all heads at once) and multiplied by a weight of that size,
 //   in front of the rotation;  q multiplied by the position's temperature 1 + tq_coef ln(floor((pos + 1) /
@@ -57,7 +58,8 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
                                                         const float* __restrict__ k_w, float eps, int rot, float base,
                                                         float lam, const float* __restrict__ v_other,
                                                         float* __restrict__ v_keep, int upr, int v_col, float tq_coef,
-                                                        int tq_every) {
+                                                        int tq_every, const double* __restrict__ rot_freq,
+                                                        float rot_amp, int rot_pairs) {
   extern __shared__ float sm[];   // [rot]: cos | sin;  [upr][D]: the heads of one round
   __shared__ float red[16];
   const int r = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
@@ -66,9 +68,9 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
   if (rot) {
     const double lb = log((double)base), p = (double)positions[r];
     for (int i = tid; i < half; i += 256) {
-      const double ang = p * exp(-(double)(2 * i) / (double)rot * lb);
-      cs[i] = (float)cos(ang);
-      cs[half + i] = (float)sin(ang);
+      const double ang = p * (rot_freq ? rot_freq[i] : exp(-(double)(2 * i) / (double)rot * lb));
+      cs[i] = (float)cos(ang) * rot_amp;
+      cs[half + i] = (float)sin(ang) * rot_amp;
     }
   }
   const int sl = slots[r];
@@ -113,7 +115,10 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
         float xv = 0.f;
         if (d < D) {
           xv = buf[d];
-          if (d < half) {
+          if (rot_pairs && d < rot) {
+            const int j = d >> 1;
+            xv = (d & 1) ? xv * cs[j] + buf[d - 1] * cs[half + j] : xv * cs[j] - buf[d + 1] * cs[half + j];
+          } else if (d < half) {
             xv = xv * cs[d] - buf[d + half] * cs[half + d];
           } else if (d < rot) {
             const int j = d - half;
@@ -147,7 +152,7 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
     if (v_keep) v_keep[(size_t)r * NV + c] = v;
     if (v_other) v = (1.f - lam) * v + lam * v_other[(size_t)r * NV + c];
     if (sl >= 0) {
-      sta(vc, (size_t)sl * NV + c, v);
+      if (vc) sta(vc, (size_t)sl * NV + c, v);
       if (vt) sta(vt, ((size_t)page * NV + c) * BS + off, v);
     }
   }
@@ -603,10 +608,10 @@ K8S_API int k8s_attn_prep(const float* qkv, int qs, const float* bias, int H, in
                           const int* slots, void* kc, void* vc, void* vt, int BS, void* q_out, int dt, int norm,
                           const float* q_w, const float* k_w, float eps, int rot, float base, float lam,
                           const float* v_other, float* v_keep, int T, hipStream_t s, int v_col, float tq_coef,
-                          int tq_every) {
+                          int tq_every, const double* rot_freq, float rot_amp, int rot_pairs) {
   if (T <= 0) return 0;
   if (H < 1 || G < 0 || D < 1 || D > 64 * kPrepPer || NV < 0 || rot < 0 || rot > D || (rot & 1) || BS < 1 ||
-      norm < 0 || norm > 2 || v_col < 0 || tq_every < 0 || ((G > 0 || NV > 0) && (!kc || !vc)))
+      norm < 0 || norm > 2 || v_col < 0 || tq_every < 0 || (G > 0 && !kc) || (NV > 0 && !vc && !vt))
     return (int)hipErrorInvalidValue;
   const int units = H + G;
   const int upr = (size_t)(rot + units * D) * sizeof(float) <= 64 * 1024 ? units : 4;    // heads per round
@@ -614,11 +619,11 @@ K8S_API int k8s_attn_prep(const float* qkv, int qs, const float* bias, int H, in
   if (dt == 0)
     hipLaunchKernelGGL((attn_prep_kernel<uint16_t>), dim3(T), dim3(256), lds, s, qkv, qs, bias, H, G, D, NV, positions,
                        slots, (uint16_t*)kc, (uint16_t*)vc, (uint16_t*)vt, BS, (uint16_t*)q_out, norm, q_w, k_w, eps, rot,
-                       base, lam, v_other, v_keep, upr, v_col, tq_coef, tq_every);
+                       base, lam, v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs);
   else
     hipLaunchKernelGGL((attn_prep_kernel<float>), dim3(T), dim3(256), lds, s, qkv, qs, bias, H, G, D, NV, positions, slots,
                        (float*)kc, (float*)vc, (float*)vt, BS, (float*)q_out, norm, q_w, k_w, eps, rot, base, lam,
-                       v_other, v_keep, upr, v_col, tq_coef, tq_every);
+                       v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs);
   return (int)hipGetLastError();
 }
 
@@ -651,7 +656,7 @@ K8S_API int k8s_masked_attn_rows(const void* q, const void* kc, const void* vc, 
 
 // 1 when the matrix-core kernel takes these sizes (bf16 only)
 K8S_API int k8s_masked_attn_mfma_ok(int H, int G, int D, int V) {
-  return H >= 1 && G >= 1 && H % G == 0 && (D == 64 || D == 128) && (V == 64 || V == 128);
+  return H >= 1 && G >= 1 && H % G == 0 && (((D == 64 || D == 128) && (V == 64 || V == 128)) || (D == 96 && V == 96));
 }
 
 K8S_API int k8s_masked_attn_mfma(const void* q, const void* kc, const void* vt, const int* block_tables, int maxb,
@@ -689,6 +694,7 @@ K8S_API int k8s_masked_attn_mfma(const void* q, const void* kc, const void* vt, 
   a.n_parts = n_parts > 1 ? n_parts : 1;
   a.pml = pml;
   a.po = po;
+  if (D == 96) return launch_mask_mfma<3, 6>(a, n_items, s);
   if (D == 64 && V == 64) return launch_mask_mfma<2, 4>(a, n_items, s);
   if (D == 64 && V == 128) return launch_mask_mfma<2, 8>(a, n_items, s);
   if (D == 128 && V == 64) return launch_mask_mfma<4, 4>(a, n_items, s);

@@ -199,7 +199,7 @@ class StepExecMixin:
         """The step in the SEGMENT layout (models with ``step_layout == "segments"``):
         consecutive rows of one sequence form a segment -- a decode token, the tokens
         of a short portion among the decode rows, or a prefill chunk -- with its first
-        position, its state slot and its block table; attention, convolutions and
+        position, its state slot (0 where the model keeps no state beside its pages) and its block table; attention, convolutions and
         recurrences all address rows through it.  Header tag 2; payload
         ids pos slots sidx | row_seg seg_row0 seg_pos0 seg_slot block_tables."""
         BS = self.kv.block_size
@@ -223,9 +223,10 @@ class StepExecMixin:
             bt[i, :len(s.blocks)] = s.blocks
             row0[i + 1] = row0[i] + q
             pos0[i] = a
-            if s.slot is None:
-                raise RuntimeError(f"sequence {s.id} runs without a state slot")
-            slot[i] = s.slot
+            if self.states is not None:
+                if s.slot is None:
+                    raise RuntimeError(f"sequence {s.id} runs without a state slot")
+                slot[i] = s.slot
             ids.extend(s.tokens[a:a + q])
             p = np.arange(a, a + q, dtype=np.int64)
             pos.append(p)
@@ -240,7 +241,7 @@ class StepExecMixin:
         header[:7] = [2, flat.size, T, n_dec_rows, n, maxb, len(sample_idx)]
         return header, flat
 
-    def _exec_segments(self, header: np.ndarray, flat_host: np.ndarray, flat_dev: torch.Tensor):
+    def _exec_segments(self, header: np.ndarray, flat_host: np.ndarray, flat_dev: torch.Tensor, spec=None):
         from ..ops.seq_ops import SegMeta, SegStepInputs
         _, _, T, n_dec_rows, n, maxb, ns = [int(v) for v in header[:7]]
         o = 0
@@ -252,6 +253,9 @@ class StepExecMixin:
             return d, h
 
         d_ids, _ = take(T)
+        if spec is not None:
+            d_ids = d_ids.clone()
+            self._apply_spec(d_ids, spec[0], _spec_tok(spec))
         d_pos, _ = take(T)
         d_slots, _ = take(T)
         d_sidx, _ = take(ns)
@@ -264,7 +268,7 @@ class StepExecMixin:
                       block_tables=bt.view(n, maxb), row0_host=row0_h.tolist(), pos0_host=pos0_h.tolist(),
                       slot_host=slot_h.tolist(), n_single=n_dec_rows)
         inp = SegStepInputs(d_ids, d_pos, d_slots, seg, d_sidx.long())
-        return self.model.forward(inp, *self.kv.tensors(), self.states.t)
+        return self.model.forward(inp, *self.kv.tensors(), self.states.t if self.states is not None else {})
 
     def _pack_step(self, decode, chunks, sample_idx):
         """``decode``: decode-attention rows (sequence, token offset past n_cached)."""
@@ -309,9 +313,9 @@ class StepExecMixin:
         from ..models.llama import StepInputs
 
         if int(header[0]) == 2:
-            if spec is not None:
-                raise RuntimeError("segment-layout steps take their tokens from the host")
-            return self._exec_segments(header, flat_host, flat_dev)
+            if spec is not None and self.stateful:
+                raise RuntimeError("stateful models take their tokens from the host")
+            return self._exec_segments(header, flat_host, flat_dev, spec)
         (_, _, T, nd, n_dec, maxb_d, n_pre, maxb_p, n_tiles, ns, n_parts, n_merge, part,
          n_items) = [int(v) for v in header]
         if self._sim:

@@ -7,8 +7,9 @@ checkpoint folder's config.json.
 * ``ligipel``             -- :class:`~.ligipel.LigipelModel` (config.json with ``"architecture": "Ligipel"``)
 * ``lizesun``             -- :class:`~.lizesun.LizesunModel` (config.json with ``"architecture": "Lizesun"``)
 * ``pumozen``             -- :class:`~.pumozen.PumozenModel` (config.json with ``"architecture": "Pumozen"``)
+* ``sunesun``             -- :class:`~.sunesun.SunesunModel` (config.json with ``"architecture": "Sunesun"``)
 
-The last four describe their layers one by one in config.json (``OWN_CONFIG``): their
+The last five describe their layers one by one in config.json (``OWN_CONFIG``): their
 configuration objects are built from it, not from a preset with overrides.
 """
 from __future__ import annotations
@@ -22,7 +23,8 @@ from . import config as C
 
 # architectures whose config.json lists the layers (``"architecture": <name>``): module, model class
 OWN_CONFIG = {"zasapel": ("zasapel", "ZasapelModel"), "ligipel": ("ligipel", "LigipelModel"),
-              "lizesun": ("lizesun", "LizesunModel"), "pumozen": ("pumozen", "PumozenModel")}
+              "lizesun": ("lizesun", "LizesunModel"), "pumozen": ("pumozen", "PumozenModel"),
+              "sunesun": ("sunesun", "SunesunModel")}
 
 
 def _module(arch: str):

@@ -93,7 +93,7 @@ _SIGS = {
     "k8s_latent_attn_rows": [P, P, P, I, P, P, P, P, I, P, I, I, I, I, I, F, I, P],
     "k8s_polynorm": [P, P, P, I, I, F, I, P],
     "k8s_glu_clamp": [P, P, I, I, F, F, F, I, P],
-    "k8s_router": [P, P, I, I, I, I, I, I, P, P, I, P, P, F, I, P, F],
+    "k8s_router": [P, P, I, I, I, I, I, I, P, P, I, P, P, F, I, P, F, I, I],
     "k8s_moe_gather": [P, P, P, P, I, I, I, I, P],
     "k8s_moe_combine_f32": [P, P, P, P, I, I, I, I, P],
     "k8s_grouped_any": [P, P, P, P, I, I, I, I, I, P],
@@ -114,7 +114,7 @@ _SIGS = {
     "k8s_add_dyt": [P, P, F, P, F, F, P, P, P, I, I, I, P],
     "k8s_embed_scale_dyt": [P, P, I, F, P, F, P, P, P, I, I, I, P],
     "k8s_relu_sq": [P, P, ctypes.c_long, I, P],
-    "k8s_attn_prep": [P, I, P, I, I, I, I, P, P, P, P, P, I, P, I, I, P, P, F, I, F, F, P, P, I, P, I, F, I],
+    "k8s_attn_prep": [P, I, P, I, I, I, I, P, P, P, P, P, I, P, I, I, P, P, F, I, F, F, P, P, I, P, I, F, I, P, F, I],
     "k8s_masked_attn_rows": [P, P, P, P, I, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, I, F, F, I, P, I, I],
     "k8s_masked_attn_mfma_ok": [I, I, I, I],
     "k8s_masked_attn_mfma": [P, P, P, P, I, P, I, P, P, I, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, P, I, I],
@@ -122,6 +122,9 @@ _SIGS = {
     "k8s_matrix_memory": [P, I, P, F, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, P, P, I, P, P, P, P],
     "k8s_head_norm_gate": [P, P, I, P, I, P, I, I, I, F, I, P, P, I, F, F],
     "k8s_ssd_scan": [P, I, P, I, I, P, I, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I, P, P, I, P, P, P],
+    "k8s_hyper_step": [P, P, I, P, P, I, P, P, P, P, F, P, I, I, I, I, P],
+    "k8s_hyper_embed": [P, P, I, F, P, I, P, P, F, P, I, I, I, P],
+    "k8s_hyper_read": [P, P, I, I, P, P, F, P, I, I, P],
     "k8s_walks": [P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, P, P, P, P],
 }
 # entry points whose C return type is not int

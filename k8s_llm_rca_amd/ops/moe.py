@@ -159,16 +159,20 @@ def _dt(t: torch.dtype) -> int:
 
 def route_direct(h: torch.Tensor, w_router: torch.Tensor, k: int, scoring: str = "sigmoid",
                  renorm: bool = False, choice_bias: Optional[torch.Tensor] = None,
-                 renorm_eps: float = 0.0, scale: float = 1.0, extra_rows: int = 0):
+                 renorm_eps: float = 0.0, scale: float = 1.0, extra_rows: int = 0,
+                 groups: Optional[Tuple[int, int]] = None):
     """Router straight from the hidden rows: fp32 logits ``h @ w_router.T``, scores by ``scoring``
     ("sigmoid" or "softmax"), the ``k`` largest (ties: lowest index), renormalised only with
     ``renorm`` (divided by their sum + ``renorm_eps``), then times ``scale``.  With ``choice_bias`` (fp32 [E])
-    the experts are chosen by score + bias while the weights are the plain scores.
+    the experts are chosen by score + bias while the weights are the plain scores.  ``groups = (count, keep)``:
+    the experts form ``count`` equal groups of neighbours, a group's score is the sum of its two largest choice
+    scores, and only experts of the ``keep`` best groups can be chosen.
     Returns (weights fp32 [T, k], ids int32 [T, k]).  With ``extra_rows`` = X the last X rows of ``w_router``
     are not experts: their fp32 logits are returned as a third result [T, X] (gates that read the same rows)."""
     T, W = h.shape
     X = int(extra_rows)
     E = w_router.shape[0] - X
+    ng, keep = (int(groups[0]), int(groups[1])) if groups else (0, 0)
     if use_hip(h):
         assert h.is_contiguous() and w_router.is_contiguous() and h.dtype == w_router.dtype
         w = torch.empty(T, k, dtype=torch.float32, device=h.device)
@@ -176,7 +180,7 @@ def route_direct(h: torch.Tensor, w_router: torch.Tensor, k: int, scoring: str =
         extra = torch.empty(T, X, dtype=torch.float32, device=h.device) if X else None
         check(lib().k8s_router(ptr(h), ptr(w_router), T, W, E, k, 0 if scoring == "sigmoid" else 1, int(renorm),
                                ptr(w), ptr(ids), _dt(h.dtype), stream_ptr(h), ptr(choice_bias), float(renorm_eps),
-                               X, ptr(extra), float(scale)), "router")
+                               X, ptr(extra), float(scale), ng, keep), "router")
         return (w, ids, extra) if X else (w, ids)
     z = h.float() @ w_router.float().t()
     extra = z[:, E:].contiguous()
@@ -184,6 +188,11 @@ def route_direct(h: torch.Tensor, w_router: torch.Tensor, k: int, scoring: str =
     s = torch.sigmoid(z) if scoring == "sigmoid" else torch.softmax(z, -1)
     # stable descending sort: equal scores keep the lower expert first
     c = s if choice_bias is None else s + choice_bias.float()
+    if ng:
+        best = c.view(T, ng, E // ng).topk(min(2, E // ng), -1).values.sum(-1)
+        kept = torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :keep]
+        open_ = torch.zeros(T, ng, dtype=torch.bool).scatter_(1, kept, True)
+        c = c.masked_fill(~open_.repeat_interleave(E // ng, 1), float("-inf"))
     order = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :k]
     w = torch.gather(s, 1, order)
     if renorm:

@@ -324,3 +324,80 @@ def relu_sq(u: torch.Tensor) -> torch.Tensor:
         check(lib().k8s_relu_sq(ptr(u), ptr(out), u.numel(), _odt(u.dtype), stream_ptr(u)), "relu_sq")
         return out
     return torch.relu(u.float()).pow(2).to(u.dtype)
+
+
+# ------------------------------------------------------------------ hyper-connections: S copies of the fp32 residual
+# (csrc/kernels/hyper_conn.hip).  ``x`` [T, S, W] fp32 holds the streams.  A sublayer reads
+# ``u = sum_s inn[s] x_s`` (RMS-normed) and its output y comes back as ``x_r <- sum_s mix[s, r] x_s + out[r] y``.
+def _rms_rows(u: torch.Tensor, w: torch.Tensor, eps: float, out_dtype) -> torch.Tensor:
+    return (u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w).to(out_dtype)
+
+
+def hyper_embed(ids: torch.Tensor, embed: torch.Tensor, scale: float, x: torch.Tensor, inn: torch.Tensor,
+                nw: torch.Tensor, eps: float, out_dtype) -> torch.Tensor:
+    """Every stream of ``x`` becomes ``embed[ids] * scale``; returns the first sublayer's input
+    ``rms(sum_s inn[s] x_s) * nw`` as activations (same pass)."""
+    T, S, W = x.shape
+    if use_hip(embed):
+        assert x.dtype == torch.float32 and x.is_contiguous() and embed.is_contiguous() and embed.shape[1] == W
+        assert ids.dtype == torch.int32 and ids.shape[0] == T and inn.dtype == nw.dtype == torch.float32
+        assert inn.numel() == S and nw.numel() == W
+        h = torch.empty(T, W, dtype=out_dtype, device=embed.device)
+        check(lib().k8s_hyper_embed(ptr(ids), ptr(embed), _odt(embed.dtype), float(scale), ptr(x), S, ptr(inn), ptr(nw),
+                                    float(eps), ptr(h), _odt(out_dtype), T, W, stream_ptr(embed)), "hyper_embed")
+        return h
+    x.copy_((embed[ids.long()].float() * scale)[:, None].expand(T, S, W))
+    return _rms_rows(torch.einsum("s,tsw->tw", inn, x), nw, eps, out_dtype)
+
+
+def hyper_step(x: torch.Tensor, y: torch.Tensor, out: torch.Tensor, mix: torch.Tensor, experts: Optional[tuple] = None,
+               inn: Optional[torch.Tensor] = None, nw: Optional[torch.Tensor] = None, eps: float = 0.0,
+               out_dtype=None) -> Optional[torch.Tensor]:
+    """In place on the streams ``x`` [T, S, W]: ``x_r <- sum_s mix[s, r] x_s + out[r] y`` (all at once from the old ones).
+    ``y``: fp32 rows [T, W], or with ``experts = (inv, w)`` the experts' output rows in expert order, joined on the way in
+    as ``sum_k w[t, k] y[inv[t K + k]]`` (``inv`` from :func:`..ops.moe.align`, ``w`` [T, K] fp32).  With ``inn, nw`` also
+    returns the next sublayer's input ``rms(sum_s inn[s] x_s) * nw`` of the new streams as activations."""
+    T, S, W = x.shape
+    read = nw is not None
+    if use_hip(x):
+        assert x.dtype == torch.float32 and x.is_contiguous() and y.is_contiguous() and y.shape[1] == W
+        assert out.dtype == mix.dtype == torch.float32 and out.numel() == S and mix.is_contiguous() and mix.numel() == S * S
+        inv, ew, K = None, None, 0
+        if experts is not None:
+            inv, ew = experts
+            K = ew.shape[1]
+            assert ew.dtype == torch.float32 and ew.is_contiguous() and ew.shape[0] == T
+            assert inv.dtype == torch.int32 and inv.numel() == T * K and y.shape[0] == T * K
+        else:
+            assert y.dtype == torch.float32 and y.shape[0] == T
+        h = None
+        if read:
+            assert inn.dtype == nw.dtype == torch.float32 and inn.numel() == S and nw.numel() == W
+            h = torch.empty(T, W, dtype=out_dtype, device=x.device)
+        check(lib().k8s_hyper_step(ptr(x), ptr(y), _odt(y.dtype), ptr(inv), ptr(ew), K, ptr(out), ptr(mix), ptr(inn),
+                                   ptr(nw), float(eps), ptr(h), _odt(out_dtype) if read else 1, T, S, W, stream_ptr(x)),
+              "hyper_step")
+        return h
+    if experts is not None:
+        inv, ew = experts
+        y = (y.float()[inv.long()].view(T, ew.shape[1], W) * ew[:, :, None]).sum(1)
+    x.copy_(torch.einsum("sr,tsw->trw", mix, x) + out[None, :, None] * y[:, None])
+    return _rms_rows(torch.einsum("s,tsw->tw", inn, x), nw, eps, out_dtype) if read else None
+
+
+def hyper_read(x: torch.Tensor, rows: Optional[torch.Tensor], nw: torch.Tensor, eps: float, out_dtype,
+               inn: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``rms(sum_s inn[s] x_s) * nw`` of the given rows (all without ``rows``) as activations; without ``inn`` the
+    plain sum of the streams."""
+    T, S, W = x.shape
+    R = T if rows is None else rows.shape[0]
+    if use_hip(x):
+        assert x.dtype == torch.float32 and x.is_contiguous() and nw.dtype == torch.float32 and nw.numel() == W
+        assert inn is None or (inn.dtype == torch.float32 and inn.numel() == S)
+        ri = None if rows is None else rows.to(torch.int32)
+        h = torch.empty(R, W, dtype=out_dtype, device=x.device)
+        check(lib().k8s_hyper_read(ptr(x), ptr(ri), R, S, ptr(inn), ptr(nw), float(eps), ptr(h), _odt(out_dtype), W,
+                                   stream_ptr(x)), "hyper_read")
+        return h
+    v = x if rows is None else x[rows.long()]
+    return _rms_rows(v.sum(1) if inn is None else torch.einsum("s,tsw->tw", inn, v), nw, eps, out_dtype)

@@ -645,13 +645,44 @@ def window_attention(qkv: torch.Tensor, H: int, G: int, D: int, V: int, kc: torc
 
 # ------------------------------------------------------------------ masked softmax attention with a prepared q / k,
 # and matrix-state recurrences (csrc/kernels/masked_attn.hip, matrix_mem.hip)
+@dataclass
+class Rope:
+    """A rotation of the first ``dims`` entries of every head: pair i turns by ``pos * freq[i]`` and cos and sin are
+    multiplied by ``amp``.  ``pairs``: pair i is the neighbouring entries 2i and 2i + 1 (else i and i + dims / 2)."""
+    dims: int
+    freq: torch.Tensor         # [dims / 2] fp64, on the model's device
+    amp: float = 1.0
+    pairs: bool = False
+
+
+def make_rope(dims: int, base: float, device, pairs: bool = False, yarn: Optional[Tuple[float, float, float, float]] = None
+              ) -> Rope:
+    """:class:`Rope` with ``freq[i] = base^(-2 i / dims)``.  ``yarn = (factor, original, fast, slow)``: a pair that turns
+    more than ``fast`` times within ``original`` positions keeps its frequency, one that turns less than ``slow`` times
+    has it divided by ``factor``, with a linear ramp over the pair index between the two, and
+    ``amp = 0.1 ln(factor) + 1``."""
+    f = torch.tensor([base ** (-2.0 * i / dims) for i in range(dims // 2)], dtype=torch.float64)
+    amp = 1.0
+    if yarn is not None:
+        factor, original, fast, slow = (float(v) for v in yarn)
+
+        def border(turns):
+            return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+        lo, hi = max(math.floor(border(fast)), 0), min(math.ceil(border(slow)), dims - 1)
+        ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        f = f / factor * ramp + f * (1.0 - ramp)
+        amp = 0.1 * math.log(factor) + 1.0
+    return Rope(dims, f.to(device), amp, pairs)
+
+
 def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D: int, V: int,
               positions: torch.Tensor, slots: torch.Tensor, kc: Optional[torch.Tensor], vc: Optional[torch.Tensor],
               out_dtype, norm=False, q_w: Optional[torch.Tensor] = None, k_w: Optional[torch.Tensor] = None,
               eps: float = 0.0, rot_dims: int = 0, rot_base: float = 10000.0, lam: float = 0.0,
               v_other: Optional[torch.Tensor] = None, v_keep: Optional[torch.Tensor] = None,
               vt: Optional[torch.Tensor] = None, maps: int = 1, v_is_k: bool = False,
-              q_temp: Optional[Tuple[float, int]] = None) -> torch.Tensor:
+              q_temp: Optional[Tuple[float, int]] = None, rope: Optional["Rope"] = None) -> torch.Tensor:
     """Between the joint projection and attention, one pass over the fp32 rows of ``qkv`` [T, H M D + G M D + G V]
     = (q | k | v) with ``M = maps`` score maps per head (q and k laid out [head][map][D]):  add ``bias`` (fp32, same
     width, optional);  rotate q and k on their first ``rot_dims`` entries per head (entry i paired with
@@ -659,10 +690,11 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
     head by its root mean square (``eps`` inside the root) and multiply by ``q_w`` / ``k_w`` [D] where given -- behind
     the rotation;  with ``norm="all"`` divide q, and k, by the root mean square of the WHOLE projection and multiply by
     ``q_w`` [H M D] / ``k_w`` [G M D] -- in front of the rotation;  with ``q_temp = (coef, every)`` multiply q by
-    ``1 + coef ln(floor((pos + 1) / every) + 1)``;  ``v_keep`` [T, G V] fp32 receives the values as projected;  with
+    ``1 + coef ln(floor((pos + 1) / every) + 1)``;  with ``rope`` (:class:`Rope`) its frequencies, pairing and amplitude
+    replace ``rot_dims`` / ``rot_base``;  ``v_keep`` [T, G V] fp32 receives the values as projected;  with
     ``v_other`` the values become ``(1 - lam) v + lam v_other``.  ``v_is_k``: there are no value columns, the values
     are the keys as projected (before norm and rotation; V = M D).  k and v go to the pages ``kc`` [pages, BS, G M D] /
-    ``vc`` [pages, BS, G V] at ``slots`` (and v to the transposed twin ``vt`` when given); q is returned [T, H M D] as
+    ``vc`` [pages, BS, G V] at ``slots`` (and v to the transposed twin ``vt`` when given, then ``vc`` may be None); q is returned [T, H M D] as
     activations.  ``G = 0``: only queries (a layer that reads another layer's pages)."""
     T = qkv.shape[0]
     HQ, GK = H * maps, G * maps
@@ -673,11 +705,14 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
     q_out = torch.empty(T, NQ, dtype=out_dtype, device=qkv.device)
     BS = kc.shape[1] if kc is not None else 1
     tq_coef, tq_every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
+    if rope is not None:
+        rot_dims = rope.dims
     if use_hip(qkv):
         assert qkv.dtype == torch.float32 and qkv.stride(1) == 1 and qkv.shape[1] == v_col + NV
         if G:
-            assert kc.is_contiguous() and vc.is_contiguous() and kc.dtype == vc.dtype == out_dtype
-            assert kc.shape[-1] == NK and vc.shape[-1] == NV
+            assert kc.is_contiguous() and kc.dtype == out_dtype and kc.shape[-1] == NK and (vc is not None or vt is not None)
+            assert vc is None or (vc.is_contiguous() and vc.dtype == out_dtype and vc.shape[-1] == NV)
+        assert rope is None or (rope.freq.dtype == torch.float64 and rope.freq.device == qkv.device)
         assert rot_dims % 2 == 0 and 0 <= rot_dims <= D
         for t, n in ((bias, v_col + NV), (q_w, NQ if mode == 2 else D), (k_w, NK if mode == 2 else D)):
             assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n)
@@ -687,7 +722,9 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
         check(lib().k8s_attn_prep(ptr(qkv), qkv.stride(0), ptr(bias), HQ, GK, D, NV, ptr(positions), ptr(slots),
                                   ptr(kc), ptr(vc), ptr(vt), BS, ptr(q_out), _dt(out_dtype), mode, ptr(q_w),
                                   ptr(k_w), float(eps), int(rot_dims), float(rot_base), float(lam), ptr(v_other),
-                                  ptr(v_keep), T, stream_ptr(qkv), v_col, tq_coef, tq_every), "attn_prep")
+                                  ptr(v_keep), T, stream_ptr(qkv), v_col, tq_coef, tq_every,
+                                  ptr(rope.freq) if rope is not None else None, rope.amp if rope is not None else 1.0,
+                                  int(rope is not None and rope.pairs)), "attn_prep")
         return q_out
     x = qkv + bias if bias is not None else qkv
     q, k, v = x[:, :NQ], x[:, NQ:NQ + NK], x[:, v_col:v_col + NV]
@@ -698,11 +735,17 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
     q, k = q.reshape(T, HQ, D), k.reshape(T, GK, D)
     if rot_dims:
         half = rot_dims // 2
-        f = torch.exp(-(2.0 * torch.arange(half, dtype=torch.float64) / rot_dims) * math.log(rot_base))
+        f = (rope.freq if rope is not None
+             else torch.exp(-(2.0 * torch.arange(half, dtype=torch.float64) / rot_dims) * math.log(rot_base)))
         ang = positions.double()[:, None] * f[None]
-        co, si = ang.cos().float()[:, None, :], ang.sin().float()[:, None, :]
+        amp = rope.amp if rope is not None else 1.0
+        co, si = ang.cos().float()[:, None, :] * amp, ang.sin().float()[:, None, :] * amp
 
         def rot(z):
+            if rope is not None and rope.pairs:
+                a, b = z[..., 0:rot_dims:2], z[..., 1:rot_dims:2]
+                ab = torch.stack([a * co - b * si, b * co + a * si], -1).flatten(-2)
+                return torch.cat([ab, z[..., rot_dims:]], -1)
             a, b = z[..., :half], z[..., half:rot_dims]
             return torch.cat([a * co - b * si, b * co + a * si, z[..., rot_dims:]], -1)
 
@@ -725,14 +768,15 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
         ok = slots >= 0
         sl = slots[ok].long()
         kc.view(-1, NK)[sl] = k.reshape(T, NK)[ok].to(kc.dtype)
-        vc.view(-1, NV)[sl] = v[ok].to(vc.dtype)
+        if vc is not None:
+            vc.view(-1, NV)[sl] = v[ok].to(vc.dtype)
         if vt is not None:
             vt[sl // BS, :, sl % BS] = v[ok].to(vt.dtype)
     q_out.copy_(q.reshape(T, NQ).to(out_dtype))
     return q_out
 
 
-def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.Tensor, vc: torch.Tensor,
+def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.Tensor, vc: Optional[torch.Tensor],
                      seg: SegMeta, scale: float, softcap: float = 0.0, chunk: int = 0, window: int = 0,
                      keep_first: int = 0, sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                      vt: Optional[torch.Tensor] = None, maps: int = 1, out_f32: bool = False) -> torch.Tensor:
@@ -743,7 +787,7 @@ def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.
     ``softcap`` > 0.  ``sink`` [H] fp32 adds ``exp(sink_h)`` to head h's denominator (no key, no value).  ``gate``
     [T, >= H] fp32 (row stride free): head h's output is multiplied by ``sigmoid(gate[t, h])``.
     Returns [T, H V].  With the transposed value pages ``vt`` (bf16, sizes of :func:`masked_mfma_ok`) the
-    matrix-core kernel runs.
+    matrix-core kernel runs and ``vc`` is not read (it may be None).
     ``maps`` = M > 1: every head has M score maps -- ``q`` is [T, H M D] and the key pages [.., G M D], both laid out
     [head][map][D]; map m of head h scores against key head ``(h // (H // G)) M + m``, has a softmax of its own and
     applies it to value head ``h // (H // G)``; the result is [T, H M V], every map's by itself (``sink`` and ``gate``
@@ -753,8 +797,9 @@ def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.
     HQ = H * maps
     out = torch.empty(T, HQ * V, dtype=torch.float32 if out_f32 else q.dtype, device=q.device)
     if use_hip(q):
-        assert q.is_contiguous() and q.shape[1] == HQ * D and kc.is_contiguous() and vc.is_contiguous()
-        assert kc.dtype == vc.dtype == q.dtype and kc.shape[-1] == G * maps * D and vc.shape[-1] == G * V and H % G == 0
+        assert q.is_contiguous() and q.shape[1] == HQ * D and kc.is_contiguous() and H % G == 0
+        assert kc.dtype == q.dtype and kc.shape[-1] == G * maps * D
+        assert vc is None or (vc.is_contiguous() and vc.dtype == q.dtype and vc.shape[-1] == G * V)
         assert seg.block_tables.is_contiguous() and chunk >= 0 and window >= 0 and keep_first >= 0
         assert sink is None or (sink.dtype == torch.float32 and sink.shape[0] == HQ)
         assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[1] >= HQ)
@@ -784,6 +829,7 @@ def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.
                                              int(keep_first), float(scale), float(softcap), stream_ptr(q), pb, n_parts,
                                              ptr(pml), ptr(po), int(maps), int(out_f32)), "masked_attn_mfma")
             return out
+        assert vc is not None          # the vector-pipe kernel reads token-major values
         check(lib().k8s_masked_attn_rows(ptr(q), ptr(kc), ptr(vc), ptr(seg.block_tables), seg.block_tables.shape[1],
                                          ptr(seg.row_seg), ptr(seg.seg_row0), ptr(seg.seg_pos0), ptr(sink), ptr(gate),
                                          gs, ptr(out), T, H, G, D, V, BS, int(chunk), int(window), int(keep_first),
