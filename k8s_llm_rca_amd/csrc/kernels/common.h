@@ -45,6 +45,12 @@ __device__ __forceinline__ uint16_t f2bf(float f) {
   return *reinterpret_cast<uint16_t*>(&h);
 }
 
+// activation 1 of the grouped GEMMs' epilogues
+__device__ __forceinline__ float relu_sq_f(float v) {
+  const float p = fmaxf(v, 0.f);
+  return p * p;
+}
+
 // RoPE of one (x[i], x[i + 64]) pair in a fixed operation order -- no choice
 // left to the compiler's contraction -- so every kernel that rotates (rope_kv,
 // the skinny and the prefill qkv GEMM epilogues) rounds identically.

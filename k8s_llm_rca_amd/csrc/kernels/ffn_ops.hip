@@ -130,20 +130,102 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_wave_barrier();
 }
 
+// One token's choice by one wave: sc [Et] logits (LDS) -> weights and experts; ch [E], gs [NG]: scratch (LDS).
+struct RouteArgs {
+  int E, X, K, mode, renorm;      // E routed experts, X rows behind them
+  float* w_out;
+  int* id_out;
+  const float* bias;
+  float renorm_eps;
+  float* extra;
+  float out_scale;
+  int NG, keep;
+};
+__device__ __forceinline__ void route_select(const RouteArgs& a, float* sc, float* ch, float* gs, int t, int lane) {
+  const int E = a.E, X = a.X, K = a.K, mode = a.mode, renorm = a.renorm, NG = a.NG, keep = a.keep;
+  float *w_out = a.w_out, *extra = a.extra;
+  int* id_out = a.id_out;
+  const float *bias = a.bias, renorm_eps = a.renorm_eps, out_scale = a.out_scale;
+  for (int x = lane; x < X; x += 64) extra[(size_t)t * X + x] = sc[E + x];
+  if (mode == 0) {
+    for (int e = lane; e < E; e += 64) sc[e] = 1.f / (1.f + expf(-sc[e]));
+  } else {
+    float m = -INFINITY, s = 0.f;
+    for (int e = lane; e < E; e += 64) m = fmaxf(m, sc[e]);
+    m = wave_max(m);
+    for (int e = lane; e < E; e += 64) s += (sc[e] = expf(sc[e] - m));
+    s = wave_sum(s);
+    for (int e = lane; e < E; e += 64) sc[e] /= s;
+  }
+  for (int e = lane; e < E; e += 64) ch[e] = bias ? sc[e] + bias[e] : sc[e];
+  wave_lds_fence();
+  if (NG > 0) {
+    const int n = E / NG;
+    for (int g = lane; g < NG; g += 64) {
+      float a = -INFINITY, b = -INFINITY;     // the two largest
+      for (int e = g * n; e < (g + 1) * n; ++e) {
+        const float v = ch[e];
+        if (v > a) {
+          b = a;
+          a = v;
+        } else {
+          b = fmaxf(b, v);
+        }
+      }
+      gs[g] = n > 1 ? a + b : a;
+    }
+    for (int k = 0; k < keep; ++k) {          // a kept group's score becomes -infinity
+      float bv = -INFINITY;
+      int bi = 1 << 30;
+      for (int g = lane; g < NG; g += 64)
+        if (gs[g] > bv) {
+          bv = gs[g];
+          bi = g;
+        }
+      wave_argmax(bv, bi);
+      if (bi < NG && (bi & 63) == lane) gs[bi] = -INFINITY;
+    }
+    wave_lds_fence();
+    for (int e = lane; e < E; e += 64)
+      if (gs[e / n] != -INFINITY) ch[e] = -INFINITY;
+  }
+  float tot = 0.f;
+  for (int k = 0; k < K; ++k) {
+    float bv = -INFINITY;
+    int bi = 1 << 30;
+    for (int e = lane; e < E; e += 64)
+      if (ch[e] > bv) {
+        bv = ch[e];
+        bi = e;
+      }
+    wave_argmax(bv, bi);
+    if (bi >= E) bi = k;                      // only where scores are not numbers: an index in range
+    const float v = sc[bi];
+    if ((bi & 63) == lane) ch[bi] = -INFINITY;
+    tot += v;
+    if (lane == 0) {
+      w_out[t * K + k] = v;
+      id_out[t * K + k] = bi;
+    }
+  }
+  if (lane == 0) {
+    if (renorm)
+      for (int k = 0; k < K; ++k) w_out[t * K + k] /= (tot + renorm_eps);
+    if (out_scale != 1.f)
+      for (int k = 0; k < K; ++k) w_out[t * K + k] *= out_scale;
+  }
+  wave_lds_fence();    // the scratch may be used for the wave's next token
+}
+
 template <typename TA, typename TW>
 __global__ void __launch_bounds__(256) router_kernel(const TA* __restrict__ h, const TW* __restrict__ wr, int T, int W,
-                                                     int Et, int K, int mode, int renorm, float* __restrict__ w_out,
-                                                     int* __restrict__ id_out, const float* __restrict__ bias,
-                                                     float renorm_eps, int X, float* __restrict__ extra,
-                                                     float out_scale, int NG, int keep) {
+                                                     RouteArgs ra) {
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int t = blockIdx.x * 4 + wv;
   if (t >= T) return;
-  float* sc = sm + wv * (2 * Et + NG);
-  float* ch = sc + Et;   // choice scores
-  float* gs = ch + Et;   // group scores
-  const int E = Et;      // rows whose logits are formed below; the routed ones are E - X
+  const int E = ra.E + ra.X;     // rows whose logits are formed
+  float* sc = sm + wv * (2 * E + ra.NG);
   if ((W & 7) == 0) {
     // 8 columns per lane and step, 16 experts at a time: the hidden row is read once per group
     for (int e0 = 0; e0 < E; e0 += 16) {
@@ -178,77 +260,51 @@ __global__ void __launch_bounds__(256) router_kernel(const TA* __restrict__ h, c
     }
   }
   wave_lds_fence();
-  {
-    const int E = Et - X;
-    for (int x = lane; x < X; x += 64) extra[(size_t)t * X + x] = sc[E + x];
-    if (mode == 0) {
-      for (int e = lane; e < E; e += 64) sc[e] = 1.f / (1.f + expf(-sc[e]));
-    } else {
-      float m = -INFINITY, s = 0.f;
-      for (int e = lane; e < E; e += 64) m = fmaxf(m, sc[e]);
-      m = wave_max(m);
-      for (int e = lane; e < E; e += 64) s += (sc[e] = expf(sc[e] - m));
-      s = wave_sum(s);
-      for (int e = lane; e < E; e += 64) sc[e] /= s;
-    }
-    for (int e = lane; e < E; e += 64) ch[e] = bias ? sc[e] + bias[e] : sc[e];
-    wave_lds_fence();
-    if (NG > 0) {
-      const int n = E / NG;
-      for (int g = lane; g < NG; g += 64) {
-        float a = -INFINITY, b = -INFINITY;     // the two largest
-        for (int e = g * n; e < (g + 1) * n; ++e) {
-          const float v = ch[e];
-          if (v > a) {
-            b = a;
-            a = v;
-          } else {
-            b = fmaxf(b, v);
-          }
-        }
-        gs[g] = n > 1 ? a + b : a;
-      }
-      for (int k = 0; k < keep; ++k) {          // a kept group's score becomes -infinity
-        float bv = -INFINITY;
-        int bi = 1 << 30;
-        for (int g = lane; g < NG; g += 64)
-          if (gs[g] > bv) {
-            bv = gs[g];
-            bi = g;
-          }
-        wave_argmax(bv, bi);
-        if (bi < NG && (bi & 63) == lane) gs[bi] = -INFINITY;
-      }
-      wave_lds_fence();
-      for (int e = lane; e < E; e += 64)
-        if (gs[e / n] != -INFINITY) ch[e] = -INFINITY;
-    }
-    float tot = 0.f;
-    for (int k = 0; k < K; ++k) {
-      float bv = -INFINITY;
-      int bi = 1 << 30;
-      for (int e = lane; e < E; e += 64)
-        if (ch[e] > bv) {
-          bv = ch[e];
-          bi = e;
-        }
-      wave_argmax(bv, bi);
-      if (bi >= E) bi = k;                      // only where scores are not numbers: an index in range
-      const float v = sc[bi];
-      if ((bi & 63) == lane) ch[bi] = -INFINITY;
-      tot += v;
-      if (lane == 0) {
-        w_out[t * K + k] = v;
-        id_out[t * K + k] = bi;
-      }
-    }
-    if (lane == 0) {
-      if (renorm)
-        for (int k = 0; k < K; ++k) w_out[t * K + k] /= (tot + renorm_eps);
-      if (out_scale != 1.f)
-        for (int k = 0; k < K; ++k) w_out[t * K + k] *= out_scale;
-    }
+  route_select(ra, sc, sc + E, sc + 2 * E, t, lane);
+}
+
+// The same for bf16 rows on the matrix cores: a workgroup takes 16 tokens, its waves a part of the width each
+// (products of bf16 are exact and summed in fp32), 16 NE router rows at a time; the parts are summed in LDS and every
+// wave then chooses for some of the tokens.  A router row is read once per 16 tokens.
+template <int NE>
+__global__ void __launch_bounds__(1024) router_mfma_kernel(const uint16_t* __restrict__ h, const uint16_t* __restrict__ wr,
+                                                          int T, int W, RouteArgs ra) {
+  extern __shared__ float sm[];
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, nw = blockDim.x >> 6;
+  const int r = lane & 15, hq = lane >> 4, t0 = blockIdx.x * 16, Et = ra.E + ra.X;
+  constexpr int EP = NE * 16;
+  float* part = sm;                                    // [nw][16][EP]
+  float* sc = sm + nw * 16 * EP;                       // [16][Et]
+  float* ch = sc + 16 * Et + wv * (Et + ra.NG);        // this wave's scratch
+  const int ks = W / nw, k0 = wv * ks + 8 * hq;
+  const uint16_t* hp = h + (size_t)min(t0 + r, T - 1) * W + k0;
+  const uint16_t* wp[NE];
+  f32x4 acc[NE];
+#pragma unroll
+  for (int n = 0; n < NE; ++n) {
+    wp[n] = wr + (size_t)min(16 * n + r, Et - 1) * W + k0;
+    acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
+#pragma unroll 4
+  for (int k = 0; k < ks; k += 32) {
+    const bf16x8 hv = *reinterpret_cast<const bf16x8*>(hp + k);
+#pragma unroll
+    for (int n = 0; n < NE; ++n)
+      acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hv, *reinterpret_cast<const bf16x8*>(wp[n] + k), acc[n], 0, 0, 0);
+  }
+#pragma unroll
+  for (int n = 0; n < NE; ++n)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[(wv * 16 + 4 * hq + i) * EP + 16 * n + r] = acc[n][i];   // token 4 hq + i, row r
+  __syncthreads();
+  for (int i = tid; i < 16 * Et; i += blockDim.x) {
+    const int tk = i / Et, e = i - tk * Et;
+    float a = 0.f;
+    for (int w = 0; w < nw; ++w) a += part[(w * 16 + tk) * EP + e];
+    sc[i] = a;
+  }
+  __syncthreads();
+  for (int tk = wv; tk < 16 && t0 + tk < T; tk += nw) route_select(ra, sc + tk * Et, ch, ch + Et, t0 + tk, lane);
 }
 
 // xp[i] = (w ? w[order[i]] : 1) * h[order[i] / K]: rows in expert order, scaled
@@ -278,12 +334,12 @@ __global__ void __launch_bounds__(256) moe_combine_f32_kernel(const TA* __restri
 
 // Grouped GEMM of any shape: rows offsets[e] .. offsets[e + 1] of a [rows][K]
 // times w[e]^T ([E][N][K]) -> out [rows][N].  64 x 64 tiles, 256 threads of
-// 4 x 4 outputs, fp32 accumulation on the vector pipes.  Tiles are numbered over
+// 4 x 4 outputs, fp32 accumulation on the vector pipes; act 1: max(., 0)^2 of every output.  Tiles are numbered over
 // the experts on the device (no host read of the offsets).
 template <typename TA, typename TW>
 __global__ void __launch_bounds__(256) grouped_any_kernel(const TA* __restrict__ a, const TW* __restrict__ w,
                                                           const int* __restrict__ offsets, TA* __restrict__ out,
-                                                          int E, int N, int K) {
+                                                          int E, int N, int K, int act) {
   __shared__ float As[16][65];
   __shared__ float Ws[16][65];
   int tile = blockIdx.x, e = 0, lo = 0, hi = 0;
@@ -329,7 +385,7 @@ __global__ void __launch_bounds__(256) grouped_any_kernel(const TA* __restrict__
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) stx(out, (size_t)m * N + n, acc[i][j]);
+      if (n < N) stx(out, (size_t)m * N + n, act == 1 ? relu_sq_f(acc[i][j]) : acc[i][j]);
     }
   }
 }
@@ -379,9 +435,29 @@ K8S_API int k8s_router(const void* h, const void* wr, int T, int W, int E, int K
   if (K < 1 || K > E || E + X > 1024 || X < 0 || (X > 0 && !extra) || NG < 0 ||
       (NG > 0 && (E % NG || keep < 1 || keep > NG || keep * (E / NG) < K)))
     return (int)hipErrorInvalidValue;
+  const RouteArgs ra{E, X, K, mode, renorm, w_out, id_out, bias, renorm_eps, extra, out_scale, NG, keep};
+  const int Et = E + X, ne = (Et + 15) / 16;
+  if (dt == 0 && ne <= 16 && ((uintptr_t)h & 15) == 0 && ((uintptr_t)wr & 15) == 0) {
+    // few tokens: as many waves per token tile as the width and LDS allow
+    const int ne2 = ne <= 1 ? 1 : ne <= 2 ? 2 : ne <= 4 ? 4 : ne <= 8 ? 8 : 16;
+    for (int nw = T <= 512 ? 16 : 4; nw >= 1; nw >>= 1) {
+      const size_t lds = 4 * ((size_t)nw * 16 * ne2 * 16 + 16 * Et + (size_t)nw * (Et + NG));
+      if (W % (32 * nw) || lds > 64 * 1024) continue;
+      const dim3 g((T + 15) / 16), b(64 * nw);
+#define K8S_RM(N_) hipLaunchKernelGGL((router_mfma_kernel<N_>), g, b, lds, s, (const uint16_t*)h, (const uint16_t*)wr, T, W, ra)
+      switch (ne2) {
+        case 1: K8S_RM(1); break;
+        case 2: K8S_RM(2); break;
+        case 4: K8S_RM(4); break;
+        case 8: K8S_RM(8); break;
+        default: K8S_RM(16); break;
+      }
+#undef K8S_RM
+      return (int)hipGetLastError();
+    }
+  }
   K8S_DT(dt, hipLaunchKernelGGL((router_kernel<TA, TW>), dim3((T + 3) / 4), dim3(256),
-                                 4 * (2 * (E + X) + NG) * sizeof(float), s, (const TA*)h, (const TW*)wr, T, W, E + X, K,
-                                 mode, renorm, w_out, id_out, bias, renorm_eps, X, extra, out_scale, NG, keep));
+                                 4 * (2 * Et + NG) * sizeof(float), s, (const TA*)h, (const TW*)wr, T, W, ra));
   return (int)hipGetLastError();
 }
 
@@ -402,10 +478,11 @@ K8S_API int k8s_moe_combine_f32(const void* y, const int* inv, const float* w, f
 }
 
 K8S_API int k8s_grouped_any(const void* a, const void* w, const int* offsets, void* out, int rows, int E, int N,
-                            int K, int dt, hipStream_t s) {
+                            int K, int dt, hipStream_t s, int act) {
   if (rows <= 0) return 0;
+  if (act < 0 || act > 1) return (int)hipErrorInvalidValue;
   const int max_tiles = (rows + 63) / 64 + E;
   K8S_DT(dt, hipLaunchKernelGGL((grouped_any_kernel<TA, TW>), dim3(max_tiles, (N + 63) / 64), dim3(256), 0, s,
-                                 (const TA*)a, (const TW*)w, offsets, (TA*)out, E, N, K));
+                                 (const TA*)a, (const TW*)w, offsets, (TA*)out, E, N, K, act));
   return (int)hipGetLastError();
 }

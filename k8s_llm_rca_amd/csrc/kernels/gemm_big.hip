@@ -154,7 +154,7 @@ __device__ __forceinline__ void set_chunk(f32x16& v, const f32x4& t) {
 template <int MODE, int SH>
 __device__ __forceinline__ int w_row(int tn, int h, int slab, int rho, int N) {
   if constexpr (SH == 16) {
-    if constexpr (MODE == 0)  // lane group g of the fragment pair <- columns 8g .. 8g+7
+    if constexpr (MODE == 0 || MODE == 3)  // lane group g of the fragment pair <- columns 8g .. 8g+7
       return tn * BN + 128 * h + 32 * slab + 8 * ((rho >> 2) & 3) + 4 * (rho >> 4) + (rho & 3);
     else if constexpr (MODE == 1)  // fragment 0: gate rows, fragment 1: the up rows of the same act columns
       return (rho >> 4 ? N : 0) + tn * 128 + 64 * h + 16 * slab + (rho & 15);
@@ -164,7 +164,7 @@ __device__ __forceinline__ int w_row(int tn, int h, int slab, int rho, int N) {
     // 32x32 accumulator: register r of lane half hh holds fragment row
     // (r & 3) + 8 (r >> 2) + 4 hh; rho -> (r, hh)
     const int r = (rho & 3) + 4 * (rho >> 3), hh = (rho >> 2) & 1;
-    if constexpr (MODE == 0)  // lane half hh <- columns 16 hh .. 16 hh + 15 (register order)
+    if constexpr (MODE == 0 || MODE == 3)  // lane half hh <- columns 16 hh .. 16 hh + 15 (register order)
       return tn * BN + 128 * h + 32 * slab + 16 * hh + r;
     else if constexpr (MODE == 1)  // registers 0-7: gate of act columns 8 hh .. +7, registers 8-15: their up rows
       return (r >= 8 ? N : 0) + tn * 128 + 64 * h + 16 * slab + 8 * hh + (r & 7);
@@ -186,7 +186,8 @@ struct RopeArgs {
 // MODE 0: plain (N output columns = W rows); MODE 1: SwiGLU (N = I output
 // act columns, W has 2I rows, I = N); MODE 2: the qkv projection with RoPE on q
 // and k and the paged K / V write in the epilogue (N = (nq + 2 nkv) 128; the
-// rope_kv_kernel's arithmetic and rounding: bit-identical to GEMM + k8s_rope_kv).
+// rope_kv_kernel's arithmetic and rounding: bit-identical to GEMM + k8s_rope_kv);
+// MODE 3 (grouped only): MODE 0 with max(., 0)^2 of every output.
 // VAR bit 0: ping-pong stagger of waves
 // 4-7; bit 1: s_setprio(1) around the MFMA clusters; bit 2: the 32x32x16 MFMA
 // (1 = the default).
@@ -196,7 +197,8 @@ __global__ void __launch_bounds__(512, 1) gemm_big_kernel(const uint16_t* __rest
                                                           int ldy, int M, int N, int K, int n_mt, int n_nt, int splits,
                                                           float* __restrict__ part, int tail_tiles, int tail_split,
                                                           float* __restrict__ tws, int* __restrict__ tick,
-                                                          const int* __restrict__ goffs, int G, RopeArgs ra) {
+                                                          const int* __restrict__ goffs, int G, RopeArgs ra,
+                                                          const int* __restrict__ rowmap, int rdiv) {
   constexpr int SH = (VAR & 4) ? 32 : 16;
   using GG = Geo<SH>;
   using acc_t = typename GG::acc_t;
@@ -244,7 +246,10 @@ __global__ void __launch_bounds__(512, 1) gemm_big_kernel(const uint16_t* __rest
       const int c = (bnd - a + BM - 1) / BM;
       if (lm < c) {
         e = gi;
-        x += (size_t)a * ldx;
+        if (rowmap)
+          rowmap += a;
+        else
+          x += (size_t)a * ldx;
         y += (size_t)a * ldy;
         M = bnd - a;
         break;
@@ -252,7 +257,7 @@ __global__ void __launch_bounds__(512, 1) gemm_big_kernel(const uint16_t* __rest
       lm -= c;
     }
     if (e < 0) return;  // past the last group's tiles (the grid is an upper bound)
-    w += (size_t)e * (MODE == 0 ? N : 2 * N) * K;
+    w += (size_t)e * (MODE == 1 ? 2 * N : N) * K;
     tm = lm;
   }
   const int m0 = tm * BM;
@@ -268,7 +273,8 @@ __global__ void __launch_bounds__(512, 1) gemm_big_kernel(const uint16_t* __rest
     const int lch = (lane & 7) ^ ((R >> 1) & 7);
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
-      xs[h][i] = x + (size_t)min(m0 + 128 * h + R, M - 1) * ldx + 8 * lch;
+      const int xr = min(m0 + 128 * h + R, M - 1);
+      xs[h][i] = x + (size_t)(rowmap ? rowmap[xr] / rdiv : xr) * ldx + 8 * lch;
       wsrc[h][i] = w + (size_t)w_row<MODE, SH>(tn, h, R >> 5, R & 31, N) * K + 8 * lch;
     }
   }
@@ -518,13 +524,13 @@ __global__ void __launch_bounds__(512, 1) gemm_big_kernel(const uint16_t* __rest
             }
           }
         }
-      } else if (MODE == 0) {
+      } else if (MODE == 0 || MODE == 3) {
         uint16_t* o = y + (size_t)m * ldy + tn * BN + 128 * qw + 32 * wc + NV * fhi;
 #pragma unroll
         for (int e = 0; e < NV; e += 8) {
           u16x8 ov;
 #pragma unroll
-          for (int c = 0; c < 8; ++c) ov[c] = f2bf(v[e + c]);
+          for (int c = 0; c < 8; ++c) ov[c] = f2bf(MODE == 3 ? relu_sq_f(v[e + c]) : v[e + c]);
           *reinterpret_cast<u16x8*>(o + e) = ov;
         }
       } else {
@@ -645,17 +651,17 @@ static int launch(const void* x, int ldx, const void* w, void* y, int ldy, int M
   const int grid = splits > 1 ? T * splits : T - tr + tr * ts;
   hipLaunchKernelGGL((gemm_big_kernel<MODE, VAR>), dim3(grid), dim3(512), 0, s, (const uint16_t*)x, ldx,
                      (const uint16_t*)w, (uint16_t*)y, ldy, M, N, K, n_mt, n_nt, splits, part, tr, ts, tws, tick,
-                     (const int*)nullptr, 0, g_rope);
+                     (const int*)nullptr, 0, g_rope, (const int*)nullptr, 1);
   return (int)hipGetLastError();
 }
 
 template <int MODE, int VAR>
 static int launch_grouped(const void* x, int ldx, const void* w, void* y, int ldy, const int* offs, int G, int R, int N,
-                          int K, hipStream_t s) {
-  const int n_mt = (R + BM - 1) / BM + G, n_nt = MODE == 0 ? N / BN : N / 128;
+                          int K, hipStream_t s, const int* rowmap, int rdiv) {
+  const int n_mt = (R + BM - 1) / BM + G, n_nt = MODE == 1 ? N / 128 : N / BN;
   hipLaunchKernelGGL((gemm_big_kernel<MODE, VAR>), dim3(n_mt * n_nt), dim3(512), 0, s, (const uint16_t*)x, ldx,
                      (const uint16_t*)w, (uint16_t*)y, ldy, R, N, K, n_mt, n_nt, 1, (float*)nullptr, 0, 1,
-                     (float*)nullptr, (int*)nullptr, offs, G, RopeArgs{});
+                     (float*)nullptr, (int*)nullptr, offs, G, RopeArgs{}, rowmap, rdiv);
   return (int)hipGetLastError();
 }
 
@@ -697,21 +703,27 @@ static int big_launch(const void* x, int ldx, const void* w, void* y, int ldy, i
 
 // Grouped (MoE experts): y rows goffs[g] .. goffs[g+1] = x rows of group g times
 // weight g (w = [G][N or 2N][K] contiguous; mode 1 = SwiGLU, y = [R][N] act).
-// R = rows of x / y (>= goffs[G]); rows past goffs[G] are never read or written.
+// mode 3 = max(., 0)^2 of every output.  R = rows of x / y (>= goffs[G]); rows past goffs[G] are never read or
+// written.  rowmap [R]: row i of the operand is x row rowmap[i] / rdiv (the permutation into expert order is read by
+// the loads, no gathered copy is made).
 K8S_API int k8s_gemm_big_grouped(const void* x, int ldx, const void* w, void* y, int ldy, const int* offs, int G, int R,
-                                 int N, int K, int mode, int var, hipStream_t s) {
+                                 int N, int K, int mode, int var, hipStream_t s, const int* rowmap, int rdiv) {
   using namespace k8s::big;
   if (R <= 0) return 0;
-  if (G <= 0 || !offs || K % (2 * BK) || ldx % 8 || ldx < K || ldy < N || N <= 0 || (mode == 0 && N % BN) ||
-      (mode == 1 && N % 128) || (mode != 0 && mode != 1) || ((uintptr_t)x % 16) || ((uintptr_t)w % 16) ||
-      (mode == 0 && (ldy % 8 || (uintptr_t)y % 16)) || (mode == 1 && (ldy % 4 || (uintptr_t)y % 8)))
+  if (G <= 0 || !offs || K % (2 * BK) || ldx % 8 || ldx < K || ldy < N || N <= 0 || (mode != 1 && N % BN) ||
+      (mode == 1 && N % 128) || (mode != 0 && mode != 1 && mode != 3) || ((uintptr_t)x % 16) || ((uintptr_t)w % 16) ||
+      (mode != 1 && (ldy % 8 || (uintptr_t)y % 16)) || (mode == 1 && (ldy % 4 || (uintptr_t)y % 8)) ||
+      (rowmap && rdiv < 1))
     return (int)hipErrorInvalidValue;
   const bool sh32 = var & 4;
   if (mode == 0)
-    return sh32 ? launch_grouped<0, 5>(x, ldx, w, y, ldy, offs, G, R, N, K, s)
-                : launch_grouped<0, 1>(x, ldx, w, y, ldy, offs, G, R, N, K, s);
-  return sh32 ? launch_grouped<1, 5>(x, ldx, w, y, ldy, offs, G, R, N, K, s)
-              : launch_grouped<1, 1>(x, ldx, w, y, ldy, offs, G, R, N, K, s);
+    return sh32 ? launch_grouped<0, 5>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv)
+                : launch_grouped<0, 1>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv);
+  if (mode == 3)
+    return sh32 ? launch_grouped<3, 5>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv)
+                : launch_grouped<3, 1>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv);
+  return sh32 ? launch_grouped<1, 5>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv)
+              : launch_grouped<1, 1>(x, ldx, w, y, ldy, offs, G, R, N, K, s, rowmap, rdiv);
 }
 
 // Split-tail workspace of the calling thread's current device: `ws` (device

@@ -387,7 +387,7 @@ __device__ __forceinline__ void glds_strip(const uint16_t* __restrict__ x, int l
 // of y (final) or fp32 rows of `part` (split-K partial), rows < M only.
 template <int MTW, int NF = 4>
 __device__ __forceinline__ void glds_store(const f32x4 (&acc)[MTW][NF], int M, uint16_t* __restrict__ y, int ldy,
-                                           float* __restrict__ pp, int ldp, bool silu = false) {
+                                           float* __restrict__ pp, int ldp, bool silu = false, int act = 0) {
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int r = lane & 15, g = lane >> 4;
   const int m_base = wv * 16 * MTW;
@@ -418,7 +418,7 @@ __device__ __forceinline__ void glds_store(const f32x4 (&acc)[MTW][NF], int M, u
           if (pp)
             pp[(size_t)m * ldp + 16 * cf + r] = acc[mt][cf][v];
           else
-            y[(size_t)m * ldy + 16 * cf + r] = f2bf(acc[mt][cf][v]);
+            y[(size_t)m * ldy + 16 * cf + r] = f2bf(act == 1 ? relu_sq_f(acc[mt][cf][v]) : acc[mt][cf][v]);
         }
       }
     }
@@ -486,7 +486,7 @@ __global__ void __launch_bounds__(256) grouped_glds_kernel(const uint16_t* __res
                                                            const uint16_t* __restrict__ w, uint16_t* __restrict__ y,
                                                            int ldy, float* __restrict__ part,
                                                            const int* __restrict__ offsets, int E, int N, int K,
-                                                           int kslice, int total_rows) {
+                                                           int kslice, int total_rows, int act) {
   __shared__ __attribute__((aligned(16))) uint16_t sm[glds_lds_elems<1, NB>()];
   int j = blockIdx.y, e = 0, row0 = 0, rows = 0;
   for (; e < E; ++e) {
@@ -507,7 +507,7 @@ __global__ void __launch_bounds__(256) grouped_glds_kernel(const uint16_t* __res
   glds_strip<1, NB>(x + (size_t)row0 * ldx + kbeg, ldx, rows, w + ((size_t)e * N + n0) * K + kbeg, K, kslice / kSC,
                     sm, acc);
   if (gridDim.z == 1)
-    glds_store<1>(acc, rows, y + (size_t)row0 * ldy + n0, ldy, nullptr, 0);
+    glds_store<1>(acc, rows, y + (size_t)row0 * ldy + n0, ldy, nullptr, 0, false, act);
   else
     glds_store<1>(acc, rows, nullptr, 0, part + ((size_t)split * total_rows + row0) * N + n0, N);
 }
@@ -757,10 +757,10 @@ K8S_API int k8s_gemm_stream_part(const void* x, int ldx, const void* w, void* y,
 // unless reduce == 0.
 static int grouped_glds_launch(const void* x, int ldx, const void* w, void* y, int ldy, const int* offsets, int E,
                                int N, int K, int max_tiles, int cfg, int splits, void* part, int total_rows,
-                               bool reduce, hipStream_t s) {
+                               bool reduce, hipStream_t s, int act = 0) {
   if (total_rows <= 0) return (int)hipSuccess;
   if (E <= 0 || N % kSBN || splits < 1 || K % (splits * kSC) || (splits > 1 && part == nullptr) || cfg < 13 ||
-      cfg > 16 || ldx % 8 || max_tiles <= 0 || (splits > 1 && ((size_t)total_rows * N) % 8))
+      cfg > 16 || ldx % 8 || max_tiles <= 0 || (splits > 1 && ((size_t)total_rows * N) % 8) || act < 0 || act > 1 || (act && splits > 1))
     return (int)hipErrorInvalidValue;
   const int kslice = K / splits;
   const dim3 grid(N / kSBN, max_tiles, splits);
@@ -770,7 +770,7 @@ static int grouped_glds_launch(const void* x, int ldx, const void* w, void* y, i
   float* pp = (float*)part;
 #define K8S_GG(NB)                                                                                               \
   hipLaunchKernelGGL((grouped_glds_kernel<NB>), grid, dim3(256), 0, s, xx, ldx, ww, yy, ldy, pp, offsets, E, N, K, \
-                     kslice, total_rows)
+                     kslice, total_rows, act)
   switch (cfg) {
     case 13: K8S_GG(3); break;
     case 14: K8S_GG(4); break;
@@ -789,6 +789,7 @@ static int grouped_glds_launch(const void* x, int ldx, const void* w, void* y, i
 }
 
 K8S_API int k8s_grouped_glds(const void* x, int ldx, const void* w, void* y, int ldy, const int* offsets, int E, int N,
-                             int K, int max_tiles, int cfg, int splits, void* part, int total_rows, hipStream_t s) {
-  return grouped_glds_launch(x, ldx, w, y, ldy, offsets, E, N, K, max_tiles, cfg, splits, part, total_rows, true, s);
+                             int K, int max_tiles, int cfg, int splits, void* part, int total_rows, hipStream_t s,
+                             int act) {
+  return grouped_glds_launch(x, ldx, w, y, ldy, offsets, E, N, K, max_tiles, cfg, splits, part, total_rows, true, s, act);
 }

@@ -11,6 +11,7 @@
 // patterns), register-staged double buffer, one barrier per k-tile.
 // v_mfma_f32_16x16x32_bf16 with A = W rows, B = X^T: each lane ends with 4
 // consecutive output columns of one row (8-byte stores).
+// act 1: max(y, 0)^2 of the whole sum (in the epilogue, or in the split-K reduce).
 // FUSE_SILU: A[m][k] = silu(G[m][k]) * U[m][k] computed while staging, with
 // G|U the gate_up output [rows][2K] (the down projection never materialises
 // the activation).
@@ -34,7 +35,7 @@ __global__ void __launch_bounds__(256, 2) grouped_gemm_kernel(const uint16_t* __
                                                               const uint16_t* __restrict__ w,
                                                               uint16_t* __restrict__ y, int ldy,
                                                               const int* __restrict__ offsets, int E, int N, int K,
-                                                              float* __restrict__ part, int total_rows) {
+                                                              float* __restrict__ part, int total_rows, int act) {
   __shared__ __attribute__((aligned(16))) uint16_t sA[2][GG_BM * GG_BK];
   __shared__ __attribute__((aligned(16))) uint16_t sB[2][GG_BN * GG_BK];
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
@@ -155,7 +156,7 @@ __global__ void __launch_bounds__(256, 2) grouped_gemm_kernel(const uint16_t* __
     for (int nt = 0; nt < 4; ++nt) {
       u16x4 v;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] = f2bf(acc[nt][mt][i]);
+      for (int i = 0; i < 4; ++i) v[i] = f2bf(act == 1 ? relu_sq_f(acc[nt][mt][i]) : acc[nt][mt][i]);
       *reinterpret_cast<u16x4*>(yr + 16 * nt) = v;
     }
   }
@@ -165,7 +166,7 @@ __global__ void __launch_bounds__(256, 2) grouped_gemm_kernel(const uint16_t* __
 __global__ void __launch_bounds__(256) grouped_reduce_kernel(const float* __restrict__ part, int splits,
                                                              uint16_t* __restrict__ y, int ldy,
                                                              const int* __restrict__ offsets, int E, int N,
-                                                             int total_rows) {
+                                                             int total_rows, int act) {
   const int used = offsets[E];
   const size_t RN = (size_t)total_rows * N;
   for (size_t idx = (size_t)(blockIdx.x * 256 + threadIdx.x) * 8; idx < (size_t)used * N;
@@ -180,8 +181,8 @@ __global__ void __launch_bounds__(256) grouped_reduce_kernel(const float* __rest
     u16x8 o;
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
-      o[v] = f2bf(a0[v]);
-      o[v + 4] = f2bf(a1[v]);
+      o[v] = f2bf(act == 1 ? relu_sq_f(a0[v]) : a0[v]);
+      o[v + 4] = f2bf(act == 1 ? relu_sq_f(a1[v]) : a1[v]);
     }
     *reinterpret_cast<u16x8*>(y + row * ldy + n) = o;
   }
@@ -196,22 +197,22 @@ using namespace k8s;
 // of `a`, >= offsets[E]); K % (64 * splits) == 0.
 static int launch_grouped(const void* a, int lda, const void* w, void* y, int ldy, const int* offsets, int E, int N,
                           int K, int max_tiles, int fuse_silu, int splits, void* part, int total_rows, bool reduce,
-                          hipStream_t s) {
+                          hipStream_t s, int act = 0) {
   if (N % GG_BN || K % (GG_BK * splits) || E <= 0 || max_tiles <= 0 || splits < 1 || (splits > 1 && !part) ||
-      N % 8 || ldy % 8)
+      N % 8 || ldy % 8 || act < 0 || act > 1)
     return (int)hipErrorInvalidValue;
   const dim3 grid(N / GG_BN, max_tiles, splits);
   float* pp = (float*)part;
   if (fuse_silu)
     hipLaunchKernelGGL(grouped_gemm_kernel<true>, grid, dim3(256), 0, s, (const uint16_t*)a, lda,
-                       (const uint16_t*)w, (uint16_t*)y, ldy, offsets, E, N, K, pp, total_rows);
+                       (const uint16_t*)w, (uint16_t*)y, ldy, offsets, E, N, K, pp, total_rows, act);
   else
     hipLaunchKernelGGL(grouped_gemm_kernel<false>, grid, dim3(256), 0, s, (const uint16_t*)a, lda,
-                       (const uint16_t*)w, (uint16_t*)y, ldy, offsets, E, N, K, pp, total_rows);
+                       (const uint16_t*)w, (uint16_t*)y, ldy, offsets, E, N, K, pp, total_rows, act);
   if (splits > 1 && reduce) {
     const int blocks = min(2048, (int)(((size_t)total_rows * N / 8 + 255) / 256));
     hipLaunchKernelGGL(grouped_reduce_kernel, dim3(max(blocks, 1)), dim3(256), 0, s, (const float*)pp, splits,
-                       (uint16_t*)y, ldy, offsets, E, N, total_rows);
+                       (uint16_t*)y, ldy, offsets, E, N, total_rows, act);
   }
   return (int)hipGetLastError();
 }
@@ -220,6 +221,13 @@ K8S_API int k8s_grouped_gemm(const void* a, int lda, const void* w, void* y, int
                              int N, int K, int max_tiles, int fuse_silu, int splits, void* part, int total_rows,
                              hipStream_t s) {
   return launch_grouped(a, lda, w, y, ldy, offsets, E, N, K, max_tiles, fuse_silu, splits, part, total_rows, true, s);
+}
+
+// the same with activation `act` of the outputs
+K8S_API int k8s_grouped_gemm_act(const void* a, int lda, const void* w, void* y, int ldy, const int* offsets, int E,
+                                 int N, int K, int max_tiles, int splits, void* part, int total_rows, int act,
+                                 hipStream_t s) {
+  return launch_grouped(a, lda, w, y, ldy, offsets, E, N, K, max_tiles, 0, splits, part, total_rows, true, s, act);
 }
 
 // splits > 1: partials [splits][total_rows][N] stay in `part` for a fused consumer

@@ -4,7 +4,7 @@
 // attn_prep:  rows of the joint projection (fp32: q [H][D] | k [G][D] | v [NV], row stride qs)
 //   + bias;  q, k rotated on their first `rot` entries per head (entry i with i + rot / 2, or with rot_pairs
 //   entry 2i with 2i + 1; angle pos * f_i with f_i = base^(-2 i / rot) or from a table of doubles, the product
-//   formed in double; cos and sin times rot_amp);  norm 1: q, k divided by the head's root mean square (eps inside
+//   formed in double; cos and sin times rot_amp; rot_cs: the step's table of them, made once for all layers);  norm 1: q, k divided by the head's root mean square (eps inside
 //   the root) behind the rotation and multiplied by a weight [D] where given;  norm 2: q and k each divided by
 //   the root mean square of the WHOLE projection (all heads at once) and multiplied by a weight of that size,
 //   in front of the rotation;  q multiplied by the position's temperature 1 + tq_coef ln(floor((pos + 1) /
@@ -59,13 +59,16 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
                                                         float lam, const float* __restrict__ v_other,
                                                         float* __restrict__ v_keep, int upr, int v_col, float tq_coef,
                                                         int tq_every, const double* __restrict__ rot_freq,
-                                                        float rot_amp, int rot_pairs) {
+                                                        float rot_amp, int rot_pairs,
+                                                        const float* __restrict__ rot_cs) {
   extern __shared__ float sm[];   // [rot]: cos | sin;  [upr][D]: the heads of one round
   __shared__ float red[16];
   const int r = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int half = rot >> 1;
   float* cs = sm;
-  if (rot) {
+  if (rot && rot_cs) {
+    for (int i = tid; i < rot; i += 256) cs[i] = rot_cs[(size_t)r * rot + i];
+  } else if (rot) {
     const double lb = log((double)base), p = (double)positions[r];
     for (int i = tid; i < half; i += 256) {
       const double ang = p * (rot_freq ? rot_freq[i] : exp(-(double)(2 * i) / (double)rot * lb));
@@ -154,6 +157,90 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(const float* __restrict_
     if (sl >= 0) {
       if (vc) sta(vc, (size_t)sl * NV + c, v);
       if (vt) sta(vt, ((size_t)page * NV + c) * BS + off, v);
+    }
+  }
+}
+
+// cs [T][2 half]: cos | sin of positions[t] * freq[j], times amp (the product in double).
+__global__ void __launch_bounds__(256) rope_table_kernel(const int* __restrict__ positions,
+                                                         const double* __restrict__ freq, float amp,
+                                                         float* __restrict__ cs, size_t n, int half) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  const size_t t = i / half;
+  const int j = (int)(i - t * half);
+  double si, co;
+  sincos((double)positions[t] * freq[j], &si, &co);
+  cs[t * 2 * half + j] = (float)co * amp;
+  cs[t * 2 * half + half + j] = (float)si * amp;
+}
+
+template <typename TA>
+__device__ __forceinline__ void sta4(TA* p, size_t i, const f32x4& v);
+template <>
+__device__ __forceinline__ void sta4<float>(float* p, size_t i, const f32x4& v) { *reinterpret_cast<f32x4*>(p + i) = v; }
+template <>
+__device__ __forceinline__ void sta4<uint16_t>(uint16_t* p, size_t i, const f32x4& v) {
+  *reinterpret_cast<u16x4*>(p + i) = u16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])};
+}
+
+// The preparation where a row's entries do not meet beyond their rotation pair (2i, 2i + 1): no norm, no bias,
+// cos | sin from the table.  A thread takes four neighbouring entries -- two pairs -- at a time straight from
+// memory to memory (no LDS).  A workgroup takes TR rows; value column c of TR rows whose slots are TR aligned
+// neighbours of one page goes to the transposed page in one store.
+template <typename TA, int TR>
+__global__ void __launch_bounds__(256) attn_prep_pairs_kernel(const float* __restrict__ x, int qs, int NQ, int NK, int NV,
+                                                              int D, int v_col, const int* __restrict__ slots,
+                                                              TA* __restrict__ kc, TA* __restrict__ vc,
+                                                              TA* __restrict__ vt, int BS, TA* __restrict__ q_out,
+                                                              int rot, const float* __restrict__ cs, int T) {
+  const int r0 = blockIdx.x * TR, tid = threadIdx.x, nv = (NQ + NK) >> 2, half = rot >> 1;
+  const int nr = min(TR, T - r0);
+  for (int i = tid; i < nr * nv; i += 256) {
+    const int rr = i / nv, c = (i - rr * nv) << 2, r = r0 + rr;
+    f32x4 v = *reinterpret_cast<const f32x4*>(x + (size_t)r * qs + c);
+    const int d = c % D;
+#pragma unroll
+    for (int k = 0; k < 4; k += 2)
+      if (d + k < rot) {
+        const float* p = cs + (size_t)r * rot + ((d + k) >> 1);
+        const float co = p[0], si = p[half], a = v[k], b = v[k + 1];
+        v[k] = a * co - b * si;
+        v[k + 1] = b * co + a * si;
+      }
+    if (c < NQ) {
+      sta4(q_out, (size_t)r * NQ + c, v);
+    } else {
+      const int sl = slots[r];
+      if (sl >= 0) sta4(kc, (size_t)sl * NK + (c - NQ), v);
+    }
+  }
+  if (NV == 0) return;
+  const int s0 = slots[r0];
+  bool run = TR > 1 && nr == TR && s0 >= 0 && s0 % TR == 0 && BS % TR == 0;    // then a page holds all TR
+  for (int k = 1; k < nr; ++k) run = run && slots[r0 + k] == s0 + k;
+  for (int c = tid; c < NV; c += 256) {
+    float v[TR];
+#pragma unroll
+    for (int k = 0; k < TR; ++k) v[k] = k < nr ? x[(size_t)(r0 + k) * qs + v_col + c] : 0.f;
+    if (vt && run) {
+      const int page = s0 / BS;
+      TA* o = vt + ((size_t)page * NV + c) * BS + (s0 - page * BS);
+#pragma unroll
+      for (int k = 0; k + 4 <= TR; k += 4) sta4(o, k, f32x4{v[k], v[k + 1], v[k + 2], v[k + 3]});
+    } else if (vt) {
+#pragma unroll
+      for (int k = 0; k < TR; ++k) {
+        const int sl = k < nr ? slots[r0 + k] : -1;
+        if (sl >= 0) sta(vt, ((size_t)(sl / BS) * NV + c) * BS + sl % BS, v[k]);
+      }
+    }
+    if (vc) {
+#pragma unroll
+      for (int k = 0; k < TR; ++k) {
+        const int sl = k < nr ? slots[r0 + k] : -1;
+        if (sl >= 0) sta(vc, (size_t)sl * NV + c, v[k]);
+      }
     }
   }
 }
@@ -608,7 +695,8 @@ K8S_API int k8s_attn_prep(const float* qkv, int qs, const float* bias, int H, in
                           const int* slots, void* kc, void* vc, void* vt, int BS, void* q_out, int dt, int norm,
                           const float* q_w, const float* k_w, float eps, int rot, float base, float lam,
                           const float* v_other, float* v_keep, int T, hipStream_t s, int v_col, float tq_coef,
-                          int tq_every, const double* rot_freq, float rot_amp, int rot_pairs) {
+                          int tq_every, const double* rot_freq, float rot_amp, int rot_pairs,
+                          const float* rot_cs) {
   if (T <= 0) return 0;
   if (H < 1 || G < 0 || D < 1 || D > 64 * kPrepPer || NV < 0 || rot < 0 || rot > D || (rot & 1) || BS < 1 ||
       norm < 0 || norm > 2 || v_col < 0 || tq_every < 0 || (G > 0 && !kc) || (NV > 0 && !vc && !vt))
@@ -619,11 +707,43 @@ K8S_API int k8s_attn_prep(const float* qkv, int qs, const float* bias, int H, in
   if (dt == 0)
     hipLaunchKernelGGL((attn_prep_kernel<uint16_t>), dim3(T), dim3(256), lds, s, qkv, qs, bias, H, G, D, NV, positions,
                        slots, (uint16_t*)kc, (uint16_t*)vc, (uint16_t*)vt, BS, (uint16_t*)q_out, norm, q_w, k_w, eps, rot,
-                       base, lam, v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs);
+                       base, lam, v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs,
+                       rot_cs);
   else
     hipLaunchKernelGGL((attn_prep_kernel<float>), dim3(T), dim3(256), lds, s, qkv, qs, bias, H, G, D, NV, positions, slots,
                        (float*)kc, (float*)vc, (float*)vt, BS, (float*)q_out, norm, q_w, k_w, eps, rot, base, lam,
-                       v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs);
+                       v_other, v_keep, upr, v_col, tq_coef, tq_every, rot_freq, rot_amp, rot_pairs,
+                       rot_cs);
+  return (int)hipGetLastError();
+}
+
+K8S_API int k8s_rope_table(const int* positions, const double* freq, float amp, float* cs, int T, int half, hipStream_t s) {
+  if (T <= 0 || half <= 0) return 0;
+  const size_t n = (size_t)T * half;
+  hipLaunchKernelGGL(rope_table_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, positions, freq, amp, cs, n,
+                     half);
+  return (int)hipGetLastError();
+}
+
+// D and qs multiples of 4, x / q_out / kc 16-byte aligned (8 for bf16 outputs); rot 0 needs no table
+K8S_API int k8s_attn_prep_pairs(const float* x, int qs, int H, int G, int D, int NV, int v_col, const int* slots,
+                                void* kc, void* vc, void* vt, int BS, void* q_out, int dt, int rot, const float* cs,
+                                int T, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (H < 1 || G < 0 || D < 4 || D % 4 || qs % 4 || rot < 0 || rot > D || rot % 2 || (rot && !cs) || NV < 0 || v_col < 0 ||
+      BS < 1 || (G > 0 && !kc) || (NV > 0 && !vc && !vt) || ((uintptr_t)x & 15))
+    return (int)hipErrorInvalidValue;
+#define K8S_PP(TA, TR)                                                                                             \
+  hipLaunchKernelGGL((attn_prep_pairs_kernel<TA, TR>), dim3((T + TR - 1) / TR), dim3(256), 0, s, x, qs, H * D, G * D, NV, \
+                     D, v_col, slots, (TA*)kc, (TA*)vc, (TA*)vt, BS, (TA*)q_out, rot, cs, T)
+  if (dt == 0) {
+    if (T > 1024) K8S_PP(uint16_t, 8);
+    else K8S_PP(uint16_t, 1);
+  } else {
+    if (T > 1024) K8S_PP(float, 8);
+    else K8S_PP(float, 1);
+  }
+#undef K8S_PP
   return (int)hipGetLastError();
 }
 

@@ -269,7 +269,7 @@ class SunesunModel:
                     L["in" + q], L["mix" + q] = f32(f"{p}hc{q}.in"), f32(f"{p}hc{q}.mix")
                     L["out" + q] = f32(f"{p}hc{q}.out") * cfg.residual_mult
                 else:                                                                  # one stream that is only added to
-                    L["in" + q], L["mix" + q], L["out" + q] = one, one, one * cfg.residual_mult
+                    L["in" + q], L["mix" + q], L["out" + q] = one, one.view(1, 1), one * cfg.residual_mult
             if f is not None:
                 m = p + "mlp."
                 L["router"] = put(m + "router")
@@ -286,12 +286,14 @@ class SunesunModel:
         """x @ w.T with an fp32 result (fp32 accumulation either way)."""
         return linear_f32out(x, w) if self.dtype == torch.bfloat16 else linear(x, w)
 
-    def _attention(self, li: int, L, h: torch.Tensor, inp: S.SegStepInputs, kc, vc, vt) -> torch.Tensor:
-        a = self.cfg.layers[li].attn
+    def _attention(self, li: int, L, h: torch.Tensor, inp: S.SegStepInputs, tables, kc, vc, vt) -> torch.Tensor:
+        a, rope = self.cfg.layers[li].attn, self.ropes[li]
         H, G, D = a.heads, a.kv_heads, a.dim
         x = self._lin32(h, L["w_in"])                                  # [T, H D + G D] fp32
-        q = S.attn_prep(x, None, H, G, D, D, inp.positions, inp.slots, kc, vc, self.dtype, rope=self.ropes[li], vt=vt,
-                        v_is_k=True)
+        if rope is not None and id(rope) not in tables:
+            tables[id(rope)] = S.rope_table(inp.positions, rope)
+        q = S.attn_prep(x, None, H, G, D, D, inp.positions, inp.slots, kc, vc, self.dtype, rope=rope,
+                        rope_cs=tables.get(id(rope)), vt=vt, v_is_k=True)
         o = S.masked_attention(q, H, G, D, D, kc, vc, inp.seg, a.scale, softcap=a.softcap, window=a.window, vt=vt)
         return self._lin32(o, L["wo"])
 
@@ -301,15 +303,17 @@ class SunesunModel:
         w, ids = M.route_direct(h, L["router"], f.top, scoring="sigmoid",
                                 groups=(f.groups, f.keep) if f.groups else None)
         order, inv, offsets = M.align(ids, f.experts)
-        xp = M.gather_rows(h, order, f.top)
-        rows = xp.shape[0]
-        dev16 = xp.is_cuda and xp.dtype == torch.bfloat16
-        if dev16 and rows <= MoELayerSet.GLDS_MAX_ROWS:
+        rows = order.numel()
+        dev16 = h.is_cuda and h.dtype == torch.bfloat16
+        if dev16 and rows > M.BIG_MIN_ROWS and M.grouped_big_ok(rows, f.ff, h.shape[1], False):
+            # prefill sizes: the grouped MFMA GEMM reads the tokens' rows in expert order itself
+            act = M.grouped_big(h, L["w_up"], offsets, act="relu_sq", order=order, k=f.top)
+        elif dev16 and rows <= MoELayerSet.GLDS_MAX_ROWS:
             # decode sizes: the weight-streaming kernels (LDS-DMA strips up; the down projection with its K split)
-            u = M.grouped_gemm(xp, L["w_up"], offsets, glds=MoELayerSet.GLDS_UP[0], splits=MoELayerSet.GLDS_UP[1])
+            act = M.grouped_gemm(M.gather_rows(h, order, f.top), L["w_up"], offsets, glds=MoELayerSet.GLDS_UP[0],
+                                 splits=MoELayerSet.GLDS_UP[1], act="relu_sq")
         else:
-            u = M.grouped_auto(xp, L["w_up"], offsets)
-        act = N.relu_sq(u)
+            act = M.grouped_auto(M.gather_rows(h, order, f.top), L["w_up"], offsets, act="relu_sq")
         if dev16 and rows <= MoELayerSet.SPLIT_MAX_ROWS:
             yp = M.grouped_gemm(act, L["w_down"], offsets, splits=MoELayerSet.DOWN_SPLITS)
         else:
@@ -324,12 +328,13 @@ class SunesunModel:
         cfg, eps, dt = self.cfg, self.cfg.norm_eps, self.dtype
         T = inp.input_ids.shape[0]
         runs = [self.weights[s] for s in self.source]
+        tables: Dict[int, torch.Tensor] = {}       # cos | sin of the step's positions, one per distinct rotation
         x = torch.empty(T, max(1, cfg.streams), cfg.hidden, dtype=torch.float32, device=self.device)
         h = N.hyper_embed(inp.input_ids, self.embed, cfg.embed_scale, x, runs[0]["in1"], runs[0]["norm1"], eps, dt)
         for li, (spec, L) in enumerate(zip(cfg.layers, runs)):
             nxt = runs[li + 1] if li + 1 < len(runs) else None
             into = dict(inn=nxt["in1"], nw=nxt["norm1"], eps=eps, out_dtype=dt) if nxt is not None else {}
-            y = self._attention(li, L, h, inp, kcs[li], vcs[li], vts[li])
+            y = self._attention(li, L, h, inp, tables, kcs[li], vcs[li], vts[li])
             if spec.mlp is None:
                 h = N.hyper_step(x, y, L["out1"], L["mix1"], **into)
             else:

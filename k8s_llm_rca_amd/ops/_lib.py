@@ -42,7 +42,7 @@ _SIGS = {
     "k8s_gemm_big": [P, I, P, P, I, I, I, I, I, I, P],
     "k8s_gemm_big_split": [P, I, P, P, I, I, I, I, I, I, P, P],
     "k8s_gemm_big_part": [P, I, P, P, I, I, I, I, I, I, P, P],
-    "k8s_gemm_big_grouped": [P, I, P, P, I, P, I, I, I, I, I, I, P],
+    "k8s_gemm_big_grouped": [P, I, P, P, I, P, I, I, I, I, I, I, P, P, I],
     "k8s_gemm_big_rope": [P, I, P, P, I, I, I, I, P, P, P, P, P, I, I, I, I, P],
     "k8s_gemm_big_ws_bytes": [],
     "k8s_gemm_big_set_ws": [P],
@@ -52,7 +52,7 @@ _SIGS = {
     "k8s_gemm_stream_silu_norm": [P, I, P, I, P, P, P, F, P, P, I, I, I, I, I, P],
     "k8s_gemm_skinny_rope_norm": [P, I, P, I, P, P, P, F, P, P, I, I, I, I, P, P, P, P, P, I, I, I, P],
     "k8s_gemm_stream_part": [P, I, P, P, I, I, I, I, I, I, P, P],
-    "k8s_grouped_glds": [P, I, P, P, I, P, I, I, I, I, I, I, P, I, P],
+    "k8s_grouped_glds": [P, I, P, P, I, P, I, I, I, I, I, I, P, I, P, I],
     "k8s_splitk_addnorm": [P, I, P, P, P, I, I, I, F, P],
     "k8s_gemm_mid_num_cfgs": [],
     "k8s_blaslt_gemm": [P, I, P, P, I, I, I, I, P, ctypes.c_size_t, P],
@@ -69,6 +69,7 @@ _SIGS = {
     "k8s_moe_align": [P, I, I, I, P, P, P, P],
     "k8s_moe_combine": [P, P, P, I, I, I, P, P],
     "k8s_grouped_gemm": [P, I, P, P, I, P, I, I, I, I, I, I, P, I, P],
+    "k8s_grouped_gemm_act": [P, I, P, P, I, P, I, I, I, I, I, P, I, I, P],
     "k8s_grouped_gemm_part": [P, I, P, P, I, P, I, I, I, I, I, I, P, I, P],
     "k8s_substr_search": [P, P, P, I, P, I, P, P, P],
     "k8s_graph_expand2": [P, P, P, P, P, P, P, P, I, I, I, I, P, P, P, P, P, P],
@@ -96,7 +97,7 @@ _SIGS = {
     "k8s_router": [P, P, I, I, I, I, I, I, P, P, I, P, P, F, I, P, F, I, I],
     "k8s_moe_gather": [P, P, P, P, I, I, I, I, P],
     "k8s_moe_combine_f32": [P, P, P, P, I, I, I, I, P],
-    "k8s_grouped_any": [P, P, P, P, I, I, I, I, I, P],
+    "k8s_grouped_any": [P, P, P, P, I, I, I, I, I, P, I],
     "k8s_layernorm": [P, P, P, P, I, I, F, I, P],
     "k8s_embed_ln": [P, P, I, P, P, P, P, P, P, I, I, I, F, P],
     "k8s_ln_residual": [P, P, P, I, P, P, P, P, P, P, P, P, I, I, I, F, P, I, P, I],
@@ -114,7 +115,9 @@ _SIGS = {
     "k8s_add_dyt": [P, P, F, P, F, F, P, P, P, I, I, I, P],
     "k8s_embed_scale_dyt": [P, P, I, F, P, F, P, P, P, I, I, I, P],
     "k8s_relu_sq": [P, P, ctypes.c_long, I, P],
-    "k8s_attn_prep": [P, I, P, I, I, I, I, P, P, P, P, P, I, P, I, I, P, P, F, I, F, F, P, P, I, P, I, F, I, P, F, I],
+    "k8s_attn_prep": [P, I, P, I, I, I, I, P, P, P, P, P, I, P, I, I, P, P, F, I, F, F, P, P, I, P, I, F, I, P, F, I, P],
+    "k8s_rope_table": [P, P, F, P, I, I, P],
+    "k8s_attn_prep_pairs": [P, I, I, I, I, I, I, P, P, P, P, I, P, I, I, P, I, P],
     "k8s_masked_attn_rows": [P, P, P, P, I, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, I, F, F, I, P, I, I],
     "k8s_masked_attn_mfma_ok": [I, I, I, I],
     "k8s_masked_attn_mfma": [P, P, P, P, I, P, I, P, P, I, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, P, I, I],

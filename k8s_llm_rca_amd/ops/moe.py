@@ -56,34 +56,45 @@ def combine(y_perm: torch.Tensor, inv: torch.Tensor, w: torch.Tensor, T: int, k:
     return out
 
 
+_ACTS = {None: 0, "relu_sq": 1}    # activations the grouped GEMMs apply to their outputs
+
+
 def grouped_gemm(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, fuse_silu: bool = False,
-                 out: Optional[torch.Tensor] = None, splits: int = 1, glds: int = 0) -> torch.Tensor:
+                 out: Optional[torch.Tensor] = None, splits: int = 1, glds: int = 0,
+                 act: Optional[str] = None) -> torch.Tensor:
     """B13: rows offsets[e]..offsets[e+1] of ``a`` times ``w[e]^T`` for every
     expert in one launch (``w`` [E, N, K]).  ``fuse_silu``: ``a`` is the
     gate_up output [rows, 2K] and the activation silu(gate) * up is formed on
     the fly.  ``splits`` > 1 splits K over workgroups (fp32 partials + a
     reduce; see grouped_gemm.hip).  ``glds`` = 10 + NB runs the LDS-DMA strip
     kernel with NB stages instead (64-row tiles: decode batches).  Offsets stay
-    on the device (no host sync)."""
+    on the device (no host sync).  ``act="relu_sq"``: ``max(y, 0)^2`` of every output, in the kernel's epilogue."""
     E, N, K = w.shape
+    code = _ACTS[act]
+    assert not (code and fuse_silu)
     rows = a.shape[0]
     if out is None:
         out = torch.empty(rows, N, dtype=a.dtype, device=a.device)
     if rows == 0:
         return out
-    if glds and use_hip(a) and a.dtype == torch.bfloat16 and not fuse_silu and N % 64 == 0 and K % (64 * splits) == 0:
+    if (glds and use_hip(a) and a.dtype == torch.bfloat16 and not fuse_silu and N % 64 == 0 and K % (64 * splits) == 0
+            and not (code and splits > 1)):
         # the LDS-DMA strip kernel (csrc/kernels/gemm_stream.hip grouped_glds_kernel)
         assert a.dtype == torch.bfloat16 and w.is_contiguous() and a.stride(1) == 1 and out.is_contiguous()
         max_tiles = (rows + 63) // 64 + E
         part = _split_scratch(a.device, splits * rows * N) if splits > 1 else None
         check(lib().k8s_grouped_glds(ptr(a), a.stride(0), ptr(w), ptr(out), out.stride(0), ptr(offsets), E, N, K,
-                                     max_tiles, glds, splits, ptr(part), rows, stream_ptr(a)), "grouped_glds")
+                                     max_tiles, glds, splits, ptr(part), rows, stream_ptr(a), code), "grouped_glds")
         return out
     if use_hip(a) and a.dtype == torch.bfloat16 and N % 128 == 0 and K % (64 * splits) == 0:
         assert a.dtype == torch.bfloat16 and w.is_contiguous() and a.stride(1) == 1 and out.is_contiguous()
         assert a.shape[1] == (2 * K if fuse_silu else K)
         max_tiles = (rows + 63) // 64 + E
         part = _split_scratch(a.device, splits * rows * N) if splits > 1 else None
+        if code:
+            check(lib().k8s_grouped_gemm_act(ptr(a), a.stride(0), ptr(w), ptr(out), out.stride(0), ptr(offsets), E, N, K,
+                                             max_tiles, splits, ptr(part), rows, code, stream_ptr(a)), "grouped_gemm_act")
+            return out
         check(lib().k8s_grouped_gemm(ptr(a), a.stride(0), ptr(w), ptr(out), out.stride(0), ptr(offsets), E, N, K,
                                      max_tiles, int(fuse_silu), splits, ptr(part), rows, stream_ptr(a)),
               "grouped_gemm")
@@ -92,7 +103,7 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, fuse_s
         # any shape, bf16 or fp32, offsets read on the device (csrc/kernels/ffn_ops.hip)
         assert w.is_contiguous() and a.is_contiguous() and out.is_contiguous() and a.shape[1] == K
         check(lib().k8s_grouped_any(ptr(a), ptr(w), ptr(offsets), ptr(out), rows, E, N, K,
-                                    0 if a.dtype == torch.bfloat16 else 1, stream_ptr(a)), "grouped_any")
+                                    0 if a.dtype == torch.bfloat16 else 1, stream_ptr(a), code), "grouped_any")
         return out
     offs = offsets.tolist()
     for e in range(E):
@@ -102,7 +113,8 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, fuse_s
         x = a[lo:hi].float()
         if fuse_silu:
             x = torch.nn.functional.silu(x[:, :K]) * x[:, K:]
-        out[lo:hi] = (x @ w[e].float().t()).to(out.dtype)
+        y = x @ w[e].float().t()
+        out[lo:hi] = (torch.relu(y).square() if code else y).to(out.dtype)
     return out
 
 
@@ -112,16 +124,22 @@ def grouped_big_ok(rows: int, N: int, K: int, silu: bool) -> bool:
 
 
 def grouped_big(x: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, silu: bool = False,
-                out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                out: Optional[torch.Tensor] = None, act: Optional[str] = None, order: Optional[torch.Tensor] = None,
+                k: int = 1) -> torch.Tensor:
     """B13 at prefill sizes on the 8-phase MFMA GEMM (csrc/kernels/gemm_big.hip,
     grouped form): rows offsets[e]..offsets[e+1] of ``x`` times ``w[e]^T`` in one
     launch with the offsets read on the device (no host sync, capturable).
     ``silu``: ``w`` [E, 2I, K] is the gate_up weight (gate rows first) and the
-    result is the SwiGLU activation [rows, I] -- gate_up is never written."""
+    result is the SwiGLU activation [rows, I] -- gate_up is never written.  ``act``: as in :func:`grouped_gemm`.
+    ``order`` (from :func:`align`, with ``k`` slots per token): ``x`` holds the TOKENS' rows and the kernel's loads read
+    row ``order[i] // k`` for row i -- no copy in expert order is made."""
     from .linear import BIG_PIPE
     E, Nw, K = w.shape
     N = Nw // 2 if silu else Nw
-    rows = x.shape[0]
+    rows = x.shape[0] if order is None else order.numel()
+    code = _ACTS[act]
+    assert not (code and silu) and (order is None or (order.dtype == torch.int32 and order.is_cuda
+                                                      and order.numel() == x.shape[0] * k))
     if out is None:
         out = torch.empty(rows, N, dtype=x.dtype, device=x.device)
     if rows == 0:
@@ -129,7 +147,8 @@ def grouped_big(x: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, silu: b
     assert x.dtype == torch.bfloat16 and w.is_contiguous() and x.stride(1) == 1 and x.shape[1] == K
     assert offsets.dtype == torch.int32 and offsets.is_cuda and grouped_big_ok(rows, N, K, silu)
     check(lib().k8s_gemm_big_grouped(ptr(x), x.stride(0), ptr(w), ptr(out), out.stride(0), ptr(offsets), E, rows, N,
-                                     K, int(silu), BIG_PIPE, stream_ptr(x)), "gemm_big_grouped")
+                                     K, 3 if code else int(silu), BIG_PIPE, stream_ptr(x), ptr(order), int(k)),
+          "gemm_big_grouped")
     return out
 
 
@@ -253,12 +272,12 @@ def combine_f32(y_perm: torch.Tensor, inv: torch.Tensor, T: int, k: int,
 BIG_MIN_ROWS = 2048   # above: the prefill-size grouped GEMM (gemm_big.hip), as the Mixtral block picks it
 
 
-def grouped_auto(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor) -> torch.Tensor:
+def grouped_auto(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, act: Optional[str] = None) -> torch.Tensor:
     """``grouped_gemm`` with the kernel chosen by size: the grouped form of the prefill GEMM for
     many rows, the weight-streaming grouped kernel for decode-size batches, the any-shape kernel
     (or fp32) otherwise.  None of them reads the offsets on the host."""
     E, N, K = w.shape
     if (use_hip(a) and a.dtype == torch.bfloat16 and a.shape[0] > BIG_MIN_ROWS
             and grouped_big_ok(a.shape[0], N, K, False)):
-        return grouped_big(a, w, offsets)
-    return grouped_gemm(a, w, offsets)
+        return grouped_big(a, w, offsets, act=act)
+    return grouped_gemm(a, w, offsets, act=act)

@@ -676,13 +676,27 @@ def make_rope(dims: int, base: float, device, pairs: bool = False, yarn: Optiona
     return Rope(dims, f.to(device), amp, pairs)
 
 
+def rope_table(positions: torch.Tensor, rope: Rope) -> torch.Tensor:
+    """[T, dims] fp32: ``amp cos(pos freq)`` | ``amp sin(pos freq)`` of a step's positions, made once for all its layers."""
+    T, half = positions.shape[0], rope.dims // 2
+    if use_hip(positions):
+        assert positions.dtype == torch.int32 and rope.freq.dtype == torch.float64 and rope.freq.device == positions.device
+        cs = torch.empty(T, rope.dims, dtype=torch.float32, device=positions.device)
+        check(lib().k8s_rope_table(ptr(positions), ptr(rope.freq), float(rope.amp), ptr(cs), T, half,
+                                   stream_ptr(positions)), "rope_table")
+        return cs
+    ang = positions.double()[:, None] * rope.freq[None]
+    return torch.cat([ang.cos().float(), ang.sin().float()], 1) * rope.amp
+
+
 def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D: int, V: int,
               positions: torch.Tensor, slots: torch.Tensor, kc: Optional[torch.Tensor], vc: Optional[torch.Tensor],
               out_dtype, norm=False, q_w: Optional[torch.Tensor] = None, k_w: Optional[torch.Tensor] = None,
               eps: float = 0.0, rot_dims: int = 0, rot_base: float = 10000.0, lam: float = 0.0,
               v_other: Optional[torch.Tensor] = None, v_keep: Optional[torch.Tensor] = None,
               vt: Optional[torch.Tensor] = None, maps: int = 1, v_is_k: bool = False,
-              q_temp: Optional[Tuple[float, int]] = None, rope: Optional["Rope"] = None) -> torch.Tensor:
+              q_temp: Optional[Tuple[float, int]] = None, rope: Optional[Rope] = None,
+              rope_cs: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Between the joint projection and attention, one pass over the fp32 rows of ``qkv`` [T, H M D + G M D + G V]
     = (q | k | v) with ``M = maps`` score maps per head (q and k laid out [head][map][D]):  add ``bias`` (fp32, same
     width, optional);  rotate q and k on their first ``rot_dims`` entries per head (entry i paired with
@@ -691,7 +705,8 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
     the rotation;  with ``norm="all"`` divide q, and k, by the root mean square of the WHOLE projection and multiply by
     ``q_w`` [H M D] / ``k_w`` [G M D] -- in front of the rotation;  with ``q_temp = (coef, every)`` multiply q by
     ``1 + coef ln(floor((pos + 1) / every) + 1)``;  with ``rope`` (:class:`Rope`) its frequencies, pairing and amplitude
-    replace ``rot_dims`` / ``rot_base``;  ``v_keep`` [T, G V] fp32 receives the values as projected;  with
+    replace ``rot_dims`` / ``rot_base`` (``rope_cs``: its :func:`rope_table` of these rows, where several layers share
+    one);  ``v_keep`` [T, G V] fp32 receives the values as projected;  with
     ``v_other`` the values become ``(1 - lam) v + lam v_other``.  ``v_is_k``: there are no value columns, the values
     are the keys as projected (before norm and rotation; V = M D).  k and v go to the pages ``kc`` [pages, BS, G M D] /
     ``vc`` [pages, BS, G V] at ``slots`` (and v to the transposed twin ``vt`` when given, then ``vc`` may be None); q is returned [T, H M D] as
@@ -719,12 +734,22 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
         for t in (v_other, v_keep):
             assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.shape == (T, NV))
         assert vt is None or (vt.is_contiguous() and vt.dtype == out_dtype and vt.shape[1:] == (NV, BS))
+        assert rope_cs is None or (rope_cs.dtype == torch.float32 and rope_cs.is_contiguous()
+                                   and rope_cs.shape == (T, rot_dims))
+        if (mode == 0 and bias is None and v_other is None and v_keep is None and not tq_every and D % 4 == 0
+                and qkv.stride(0) % 4 == 0 and qkv.data_ptr() % 16 == 0
+                and (rot_dims == 0 or (rope is not None and rope.pairs and rope_cs is not None))):
+            # nothing couples a row's entries beyond their rotation pair: memory to memory
+            check(lib().k8s_attn_prep_pairs(ptr(qkv), qkv.stride(0), HQ, GK, D, NV, v_col, ptr(slots), ptr(kc), ptr(vc),
+                                            ptr(vt), BS, ptr(q_out), _dt(out_dtype), int(rot_dims), ptr(rope_cs), T,
+                                            stream_ptr(qkv)), "attn_prep_pairs")
+            return q_out
         check(lib().k8s_attn_prep(ptr(qkv), qkv.stride(0), ptr(bias), HQ, GK, D, NV, ptr(positions), ptr(slots),
                                   ptr(kc), ptr(vc), ptr(vt), BS, ptr(q_out), _dt(out_dtype), mode, ptr(q_w),
                                   ptr(k_w), float(eps), int(rot_dims), float(rot_base), float(lam), ptr(v_other),
                                   ptr(v_keep), T, stream_ptr(qkv), v_col, tq_coef, tq_every,
                                   ptr(rope.freq) if rope is not None else None, rope.amp if rope is not None else 1.0,
-                                  int(rope is not None and rope.pairs)), "attn_prep")
+                                  int(rope is not None and rope.pairs), ptr(rope_cs)), "attn_prep")
         return q_out
     x = qkv + bias if bias is not None else qkv
     q, k, v = x[:, :NQ], x[:, NQ:NQ + NK], x[:, v_col:v_col + NV]
@@ -735,11 +760,12 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
     q, k = q.reshape(T, HQ, D), k.reshape(T, GK, D)
     if rot_dims:
         half = rot_dims // 2
-        f = (rope.freq if rope is not None
-             else torch.exp(-(2.0 * torch.arange(half, dtype=torch.float64) / rot_dims) * math.log(rot_base)))
-        ang = positions.double()[:, None] * f[None]
-        amp = rope.amp if rope is not None else 1.0
-        co, si = ang.cos().float()[:, None, :] * amp, ang.sin().float()[:, None, :] * amp
+        if rope is None:
+            f = torch.exp(-(2.0 * torch.arange(half, dtype=torch.float64) / rot_dims) * math.log(rot_base))
+            rope_cs = rope_table(positions, Rope(rot_dims, f))
+        elif rope_cs is None:
+            rope_cs = rope_table(positions, rope)
+        co, si = rope_cs[:, None, :half], rope_cs[:, None, half:]
 
         def rot(z):
             if rope is not None and rope.pairs:

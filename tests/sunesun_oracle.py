@@ -127,7 +127,10 @@ def forward(t, cfg, ids, layers_out=None):
     S = cfg.get("streams")
     xs = x[None].repeat(S or 1, 1, 1)
     for i, L in enumerate(cfg["layers"]):
-        p = f"l{L.get('weights_of', i)}."
+        j = i
+        while "weights_of" in cfg["layers"][j]:
+            j = cfg["layers"][j]["weights_of"]
+        p = f"l{j}."
         steps = [(1, lambda h: attention(t, p + "mix.", L["mixer"], h))]
         if L.get("mlp") is not None:
             steps.append((2, lambda h: feed_forward(t, p + "mlp.", L["mlp"], h)))
