@@ -36,7 +36,8 @@ __device__ __forceinline__ int rope_row(int n, int b) {  // W / output row of st
 
 // NORM: X = rmsnorm(nin) computed by the block itself into LDS (norm_prologue.h;
 // M <= kNormMaxRows, K == nin.H), after the first U weight loads are issued.
-template <int MT, int U, int NW, bool ROPE, bool NORM = false>
+// F32: y is fp32 (ldy counts floats).
+template <int MT, int U, int NW, bool ROPE, bool NORM = false, bool F32 = false>
 __global__ void __launch_bounds__(NW * 64) gemm_skinny_kernel(const uint16_t* __restrict__ x, int ldx,
                                                               const uint16_t* __restrict__ w,
                                                               uint16_t* __restrict__ y, int ldy, int M, int N, int K,
@@ -166,7 +167,10 @@ __global__ void __launch_bounds__(NW * 64) gemm_skinny_kernel(const uint16_t* __
       float v = 0.f;
 #pragma unroll
       for (int q = 0; q < NW; ++q) v += red[q][n][m];
-      y[(size_t)m * ldy + n0 + n] = f2bf(v);
+      if constexpr (F32)
+        reinterpret_cast<float*>(y)[(size_t)m * ldy + n0 + n] = v;
+      else
+        y[(size_t)m * ldy + n0 + n] = f2bf(v);
     }
   }
 }
@@ -191,6 +195,20 @@ K8S_API int k8s_gemm_skinny(const void* x, int ldx, const void* w, void* y, int 
     hipLaunchKernelGGL((gemm_skinny_kernel<4, 2, 8, false>), g, dim3(512), 0, s, xx, ldx, ww, yy, ldy, M, N, K, rp);
   else
     hipLaunchKernelGGL((gemm_skinny_kernel<8, 1, 8, false>), g, dim3(512), 0, s, xx, ldx, ww, yy, ldy, M, N, K, rp);
+  return (int)hipGetLastError();
+}
+
+// the same with an fp32 result (M <= 32)
+K8S_API int k8s_gemm_skinny_f32(const void* x, int ldx, const void* w, float* y, int ldy, int M, int N, int K,
+                                hipStream_t s) {
+  if (M <= 0 || M > 32 || N % 16 || K % 256 || ldx % 8) return (int)hipErrorInvalidValue;
+  const SkinnyRope rp{};
+  if (M <= 16)
+    hipLaunchKernelGGL((gemm_skinny_kernel<1, 4, 8, false, false, true>), dim3(N / 16), dim3(512), 0, s,
+                       (const uint16_t*)x, ldx, (const uint16_t*)w, (uint16_t*)y, ldy, M, N, K, rp);
+  else
+    hipLaunchKernelGGL((gemm_skinny_kernel<2, 4, 8, false, false, true>), dim3(N / 16), dim3(512), 0, s,
+                       (const uint16_t*)x, ldx, (const uint16_t*)w, (uint16_t*)y, ldy, M, N, K, rp);
   return (int)hipGetLastError();
 }
 

@@ -32,7 +32,7 @@ import torch
 from ..ops import moe as M
 from ..ops import norm as N
 from ..ops import seq_ops as S
-from ..ops.linear import linear, linear_f32out
+from ..ops.linear import proj_f32out
 from ..parallel.groups import ParallelContext, single
 from .moe import MoELayerSet
 
@@ -282,20 +282,16 @@ class SunesunModel:
         return sum(t.numel() * t.element_size() for t in ts)
 
     # -------------------------------------------------------------- forward
-    def _lin32(self, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-        """x @ w.T with an fp32 result (fp32 accumulation either way)."""
-        return linear_f32out(x, w) if self.dtype == torch.bfloat16 else linear(x, w)
-
     def _attention(self, li: int, L, h: torch.Tensor, inp: S.SegStepInputs, tables, kc, vc, vt) -> torch.Tensor:
         a, rope = self.cfg.layers[li].attn, self.ropes[li]
         H, G, D = a.heads, a.kv_heads, a.dim
-        x = self._lin32(h, L["w_in"])                                  # [T, H D + G D] fp32
+        x = proj_f32out(h, L["w_in"])                                  # [T, H D + G D] fp32
         if rope is not None and id(rope) not in tables:
             tables[id(rope)] = S.rope_table(inp.positions, rope)
         q = S.attn_prep(x, None, H, G, D, D, inp.positions, inp.slots, kc, vc, self.dtype, rope=rope,
                         rope_cs=tables.get(id(rope)), vt=vt, v_is_k=True)
         o = S.masked_attention(q, H, G, D, D, kc, vc, inp.seg, a.scale, softcap=a.softcap, window=a.window, vt=vt)
-        return self._lin32(o, L["wo"])
+        return proj_f32out(o, L["wo"])
 
     def _moe(self, li: int, L, h: torch.Tensor):
         """The experts' output rows in expert order, and (inv, w) that join them."""
@@ -343,7 +339,7 @@ class SunesunModel:
                 h = N.hyper_step(x, yp, L["out2"], L["mix2"], experts=join, **into)
             if layers_out is not None:
                 layers_out.append(x.sum(1))
-        return self._lin32(N.hyper_read(x, inp.logits_idx, self.final_norm, eps, dt), self.head)
+        return proj_f32out(N.hyper_read(x, inp.logits_idx, self.final_norm, eps, dt), self.head)
 
 
 def random_tensors(cfg: SunesunConfig, seed: int = 0, device="cpu") -> Dict[str, torch.Tensor]:

@@ -130,6 +130,25 @@ def linear_f32out(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return x.float() @ w.float().t()
 
 
+SKINNY_F32_MAX_M = 32
+
+
+def proj_f32out(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """``x @ w.T`` with an fp32 result: bf16 operands with fp32 accumulation (the weight-streaming kernel for a few rows,
+    hipBLASLt otherwise), or fp32 throughout."""
+    if not x.is_cuda or x.dtype != torch.bfloat16:
+        return linear(x, w)
+    M, K = x.shape
+    N = w.shape[0]
+    if (_enabled and 0 < M <= SKINNY_F32_MAX_M and N * K <= SKINNY_MAX_NK and K % 256 == 0 and N % 16 == 0
+            and x.stride(1) == 1 and x.stride(0) % 8 == 0 and w.dtype == torch.bfloat16 and w.is_contiguous()):
+        out = torch.empty((M, N), dtype=torch.float32, device=x.device)
+        check(lib().k8s_gemm_skinny_f32(ptr(x), x.stride(0), ptr(w), ptr(out), N, M, N, K, stream_ptr(x)),
+              "gemm_skinny_f32")
+        return out
+    return linear_f32out(x, w)
+
+
 def reserve_lib_workspace(dev: torch.device, claim_stream: int = None) -> None:
     """Allocate the hipBLASLt workspace (and gemm_big's split-tail workspace)
     before any HIP-graph capture.  ``claim_stream`` (a raw hipStream_t): the

@@ -495,6 +495,19 @@ def test_squared_relu_in_the_grouped_products(backend, rows, E, F, W, form):
     close(got, want, dt)
 
 
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("T", [1, 7, 16, 17, 32, 33])
+@pytest.mark.parametrize("F,W", [(48, 256), (96, 1024), (10, 24)])
+def test_projection_with_fp32_result(backend, T, F, W):
+    """A few rows on the weight-streaming kernel, more on the library's; sizes that neither splits evenly."""
+    from k8s_llm_rca_amd.ops.linear import proj_f32out
+    dev, dt = backend
+    x, w = b16(T, W, seed=1), b16(F, W, seed=2, std=W ** -0.5)
+    got = proj_f32out(x.to(dev).to(dt), w.to(dev).to(dt))
+    assert got.dtype == torch.float32
+    close(got, x @ w.T, torch.float32)
+
+
 # ------------------------------------------------------------------ whole models
 @pytest.mark.parametrize("backend", BACKENDS)
 def test_streams_match_after_every_layer(backend):
