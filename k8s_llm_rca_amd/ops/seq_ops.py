@@ -836,15 +836,17 @@ def masked_attention(q: torch.Tensor, H: int, G: int, D: int, V: int, kc: torch.
             n_items = items.shape[0]
             # steps of few rows (decoding): a tile's key blocks are split over workgroups as well -- parts of
             # MASK_PART_BLOCKS blocks of the tile's own block list (at most MASK_MAX_PARTS parts), then a merge
+            # (more tiles than that only where they are single tokens: a prompt's parts would be all traffic)
             n_parts, pb, pml, po = 1, MASK_PART_BLOCKS, None, None
-            if n_items <= WINDOW_SPLIT_ITEMS:
+            if n_items <= WINDOW_SPLIT_ITEMS or (n_items <= 4 * WINDOW_SPLIT_ITEMS and T <= 2 * n_items):
                 kmax = max(p + b - a for p, a, b in zip(seg.pos0_host, seg.row0_host[:-1], seg.row0_host[1:]))
                 nblk = -(-kmax // 32) + 1                  # an upper bound of any tile's blocks
                 if window > 0:     # a tile's span: the window, its 16 tokens, a block's alignment; + the kept blocks
                     nblk = min(nblk, (int(window) + 45) // 32 + 1 + -(-int(keep_first) // 32))
                 if chunk > 0:
                     nblk = min(nblk, (int(chunk) + 45) // 32 + 1)
-                pb = max(MASK_PART_BLOCKS, -(-nblk // MASK_MAX_PARTS))
+                most = MASK_MAX_PARTS if n_items <= WINDOW_SPLIT_ITEMS else max(1, 1024 // n_items)
+                pb = max(MASK_PART_BLOCKS, -(-nblk // most))
                 n_parts = -(-nblk // pb)
                 if n_parts > 1:
                     pml = scratch(n_items * n_parts * HQ * 32, torch.float32, q.device)

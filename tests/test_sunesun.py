@@ -403,6 +403,21 @@ def test_window_and_cap_on_the_matrix_cores(backend, H, G, D, cap, window, split
     close(got, torch.cat([want[n - 5:], want[100:]]), dt)
 
 
+@pytest.mark.parametrize("backend", MFMA_BACKEND)
+@pytest.mark.parametrize("n_seq,window", [(40, 100), (100, 0), (140, 100)])
+def test_many_decoding_sequences_on_the_matrix_cores(backend, n_seq, window):
+    """Single tokens of many sequences in one step (their key blocks split over workgroups up to a point), each at
+    another position."""
+    dev, dt = backend
+    H, G, D, n, BS = 4, 2, 128, 330, 32
+    q, k, v, kc, vc, vt, bt = attention_case(dev, dt, H, G, D, n, BS, seed=5, twin=True)
+    want = O.attend(q, k, v, 0.3, 5.0, window).reshape(n, -1)
+    at = [(37 * i + 5) % n for i in range(n_seq)]
+    got = S.masked_attention(q.reshape(n, -1)[at].to(dev).to(dt).contiguous(), H, G, D, D, kc, vc,
+                             seg_meta([1] * n_seq, at, dev, bt * n_seq), 0.3, softcap=5.0, window=window, vt=vt)
+    close(got, want[at], dt)
+
+
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("window,aim", [(0, 1), (70, "in"), (70, "out"), (33, "in"), (33, "out"), (64, "in"), (64, "out"),
                                         (1, "in"), (1, "out"), (0, 255), (0, 256), (0, 301)])
