@@ -7,6 +7,8 @@
 // The output of a mixture of experts is joined on the way in: y = sum_k w[t][k] yp[inv[t K + k]], the rows of
 // the experts' outputs in expert order, so the joined fp32 row is never written.
 // S = 1 with in = mix = 1 is the plain pre-norm residual.
+// A step may also add the embedding output once more on the way (x_r += escale * embed[eid[t]] for every stream):
+// stacks of layers that run several times in a row read it again in front of every further pass.
 //
 // One workgroup per row; a thread owns VEC neighbouring columns of all streams, so the S x S mix is in
 // registers; the row of u stays in LDS between the sum of squares and the output.
@@ -66,19 +68,22 @@ constexpr int kMaxStreams = 16;   // the form for any count: one column per thre
 // S streams at compile time (S > 0) or S_ <= kMaxStreams of them (S == 0).
 // y: fp32 rows [T][W], or (inv given) rows of yp in expert order weighted by ew [T][K].
 // out / mix: this sublayer's; in / nw: the next one's (h null: nothing reads the streams next).
+// eid (optional) [T]: token ids whose rows of emb, times es, are added to every stream.
 template <int S, int VEC, typename TY, typename TA>
 __global__ void __launch_bounds__(1024) hyper_step_kernel(float* __restrict__ x, const TY* __restrict__ y,
                                                          const int* __restrict__ inv, const float* __restrict__ ew,
                                                          int K, const float* __restrict__ out,
                                                          const float* __restrict__ mix, const float* __restrict__ in,
                                                          const float* __restrict__ nw, float eps, TA* __restrict__ h,
-                                                         int W, int S_) {
+                                                         int W, int S_, const int* __restrict__ eid,
+                                                         const TA* __restrict__ emb, float es) {
   extern __shared__ float u[];
   __shared__ float red[16];
   constexpr int SM = S > 0 ? S : kMaxStreams;
   const int n = S > 0 ? S : S_;
   const size_t t = blockIdx.x, o = t * W;
   float* xr = x + o * n;
+  const size_t e0 = eid ? (size_t)eid[t] * W : 0;
   float ss = 0.f;
   for (int c = threadIdx.x * VEC; c < W; c += blockDim.x * VEC) {
     float xv[SM][VEC], yv[VEC];
@@ -98,9 +103,10 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(float* __restrict__ x,
     } else {
       ldv<VEC>(y, o + c, yv);
     }
-    float uv[VEC];
+    float uv[VEC], av[VEC];
 #pragma unroll
-    for (int k = 0; k < VEC; ++k) uv[k] = 0.f;
+    for (int k = 0; k < VEC; ++k) uv[k] = av[k] = 0.f;
+    if (eid) ldv<VEC>(emb, e0 + c, av);
 #pragma unroll
     for (int r = 0; r < SM; ++r)
       if (r < n) {
@@ -115,6 +121,10 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(float* __restrict__ x,
 #pragma unroll
             for (int k = 0; k < VEC; ++k) nv[k] = fmaf(m, xv[s][k], nv[k]);
           }
+        if (eid) {
+#pragma unroll
+          for (int k = 0; k < VEC; ++k) nv[k] = fmaf(es, av[k], nv[k]);
+        }
         stv<VEC>(xr, (size_t)r * W + c, nv);
         if (h) {
           const float ir = in[r];
@@ -200,11 +210,11 @@ static bool hyper_row_ok(int W) { return W > 0 && (size_t)W * sizeof(float) <= 6
 template <int VEC, typename TY, typename TA>
 static void hyper_step_launch(float* x, const void* y, const int* inv, const float* ew, int K, const float* out,
                               const float* mix, const float* in, const float* nw, float eps, void* h, int T, int S,
-                              int W, hipStream_t s) {
+                              int W, const int* eid, const void* emb, float es, hipStream_t s) {
   const dim3 g(T), b(hyper_threads(T, W, VEC));
 #define K8S_HS(SS)                                                                                              \
   hipLaunchKernelGGL((hyper_step_kernel<SS, VEC, TY, TA>), g, b, W * sizeof(float), s, x, (const TY*)y, inv, ew, K, \
-                     out, mix, in, nw, eps, (TA*)h, W, S)
+                     out, mix, in, nw, eps, (TA*)h, W, S, eid, (const TA*)emb, es)
   switch (S) {
     case 1: K8S_HS(1); break;
     case 2: K8S_HS(2); break;
@@ -219,23 +229,23 @@ static void hyper_step_launch(float* x, const void* y, const int* inv, const flo
 
 using namespace k8s;
 
-// ydt / hdt / edt: 0 bf16, 1 fp32.  inv null: y is fp32 [T][W].
+// ydt / hdt / edt: 0 bf16, 1 fp32.  inv null: y is fp32 [T][W].  emb has the type of h.
 K8S_API int k8s_hyper_step(float* x, const void* y, int ydt, const int* inv, const float* ew, int K, const float* out,
                            const float* mix, const float* in, const float* nw, float eps, void* h, int hdt, int T, int S,
-                           int W, hipStream_t s) {
+                           int W, hipStream_t s, const int* eid, const void* emb, float es) {
   if (T <= 0) return 0;
   if (!hyper_row_ok(W) || S < 1 || S > kMaxStreams || !y || !out || !mix || (h && (!in || !nw)) ||
-      (inv && (!ew || K < 1)) || (!inv && ydt != 1))
+      (inv && (!ew || K < 1)) || (!inv && ydt != 1) || (eid && !emb))
     return (int)hipErrorInvalidValue;
 #define K8S_HY(VEC)                                                                                               \
   if (ydt == 0 && hdt == 0)                                                                                       \
-    hyper_step_launch<VEC, uint16_t, uint16_t>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, s);             \
+    hyper_step_launch<VEC, uint16_t, uint16_t>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, eid, emb, es, s);             \
   else if (ydt == 0)                                                                                              \
-    hyper_step_launch<VEC, uint16_t, float>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, s);                \
+    hyper_step_launch<VEC, uint16_t, float>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, eid, emb, es, s);                \
   else if (hdt == 0)                                                                                              \
-    hyper_step_launch<VEC, float, uint16_t>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, s);                \
+    hyper_step_launch<VEC, float, uint16_t>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, eid, emb, es, s);                \
   else                                                                                                            \
-    hyper_step_launch<VEC, float, float>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, s)
+    hyper_step_launch<VEC, float, float>(x, y, inv, ew, K, out, mix, in, nw, eps, h, T, S, W, eid, emb, es, s)
   if (W % 4 == 0 && S <= 4) {
     K8S_HY(4);
   } else {

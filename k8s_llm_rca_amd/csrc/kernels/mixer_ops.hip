@@ -416,14 +416,16 @@ __global__ void __launch_bounds__(256) retention_rope_kernel(float* __restrict__
   }
 }
 
+// The scan of step 2 by itself is linear attention with one decay per head (k8s_decay_attn): rows of x (TA,
+// stride xs) = q [H][D] | k [H][D] | v [H][V], with SILU each of them through z sigmoid(z) first.
 constexpr int kRetTb = 16;    // tokens per batch
 // MODE 0: blockIdx.x = segment, from the slot's state (or zero at position 0) to the slot's state.
 // Long segments are cut into chunks ([n][4]: segment, first row, rows, -) that run in parallel:
 // MODE 1: a chunk from a zero state, its end state goes to cs [chunks][H][D][V], no output;
 // (retention_carry_kernel then turns cs into every chunk's START state and advances the slot's state)
 // MODE 2: the chunk again from its start state, writing o.
-template <int DPT, int MODE>
-__global__ void __launch_bounds__(256) retention_scan_kernel(const float* __restrict__ qkvg, int qs,
+template <int DPT, int MODE, typename TA, bool SILU>
+__global__ void __launch_bounds__(256) retention_scan_kernel(const TA* __restrict__ qkvg, int qs,
                                                              const float* __restrict__ decay, float* __restrict__ state,
                                                              const int* __restrict__ seg_row0,
                                                              const int* __restrict__ seg_pos0,
@@ -465,13 +467,15 @@ __global__ void __launch_bounds__(256) retention_scan_kernel(const float* __rest
     __syncthreads();
     for (int e = tid; e < nb * D; e += 256) {
       const int tb = e / D, d = e - tb * D;
-      const float* row = qkvg + (size_t)(t0 + tb) * qs;
-      sq[e] = row[hh * D + d];
-      sk[e] = row[(H + hh) * D + d];
+      const size_t row = (size_t)(t0 + tb) * qs;
+      const float qv = ldm(qkvg, row + hh * D + d), kv = ldm(qkvg, row + (H + hh) * D + d);
+      sq[e] = SILU ? DecayExp<TA>::silu(qv) : qv;
+      sk[e] = SILU ? DecayExp<TA>::silu(kv) : kv;
     }
     for (int e = tid; e < nb * VBS; e += 256) {
       const int tb = e / VBS, vv = e - tb * VBS;
-      sv[e] = v0 + vv < V ? qkvg[(size_t)(t0 + tb) * qs + 2 * H * D + hh * V + v0 + vv] : 0.f;
+      const float xv = v0 + vv < V ? ldm(qkvg, (size_t)(t0 + tb) * qs + 2 * H * D + hh * V + v0 + vv) : 0.f;
+      sv[e] = SILU ? DecayExp<TA>::silu(xv) : xv;
     }
     __syncthreads();
     if (dg < NDG) {
@@ -682,25 +686,22 @@ K8S_API int k8s_ssd_scan(const void* x, int xs, const void* bc, int bs, int dt, 
   return (int)hipGetLastError();
 }
 
-K8S_API int k8s_retention(float* qkvg, int qs, const int* positions, const float* decay, float* state,
-                          const int* seg_row0, const int* seg_pos0, const int* seg_slot, void* out, int n_seg, int H,
-                          int D, int V, int rot, float base, float eps, int odt, hipStream_t s, int T, float* oraw,
-                          const int* chunks, int n_chunks, const int* seg_chunk0, float* cs) {
-  if (n_seg <= 0 || T <= 0) return 0;
-  if (V < 1 || rot < 0 || rot > D || (rot & 1)) return (int)hipErrorInvalidValue;
+// The scan: token by token, or (chunks given) the two chunk passes around the carry.
+template <typename TA, bool SILU>
+static int launch_decay_scan(const TA* x, int xs, const float* decay, float* state, const int* seg_row0,
+                             const int* seg_pos0, const int* seg_slot, float* oraw, int n_seg, int H, int D, int V,
+                             hipStream_t s, const int* chunks, int n_chunks, const int* seg_chunk0, float* cs) {
   const int VBS = V < 32 ? V : 32, NDG = 256 / VBS, dpt = (D + NDG - 1) / NDG;
   if (dpt > 64) return (int)hipErrorInvalidValue;
   const size_t lds = (size_t)kRetTb * (2 * D + VBS + NDG * VBS) * sizeof(float);
-  if (lds > 160 * 1024 || (size_t)rot * sizeof(float) > 64 * 1024) return (int)hipErrorInvalidValue;
-  hipLaunchKernelGGL(retention_rope_kernel, dim3(T), dim3(256), rot * sizeof(float) + 8, s, qkvg, qs, positions, H, D,
-                     rot, base);
+  if (lds > 160 * 1024) return (int)hipErrorInvalidValue;
   const int vb = (V + VBS - 1) / VBS;
 #define K8S_RET_M(DP, MODE, items)                                                                              \
   {                                                                                                             \
-    auto k = retention_scan_kernel<DP, MODE>;                                                                   \
+    auto k = retention_scan_kernel<DP, MODE, TA, SILU>;                                                         \
     if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)) \
       return (int)hipGetLastError();                                                                            \
-    hipLaunchKernelGGL(k, dim3(items, H, vb), dim3(256), lds, s, qkvg, qs, decay, state, seg_row0, seg_pos0,    \
+    hipLaunchKernelGGL(k, dim3(items, H, vb), dim3(256), lds, s, x, xs, decay, state, seg_row0, seg_pos0,       \
                        seg_slot, oraw, H, D, V, VBS, chunks, cs);                                               \
   }
 #define K8S_RET(DP)                                                                                             \
@@ -725,6 +726,37 @@ K8S_API int k8s_retention(float* qkvg, int qs, const int* positions, const float
   }
 #undef K8S_RET
 #undef K8S_RET_M
+  return (int)hipGetLastError();
+}
+
+// dt: the type of x (0 bf16, 1 fp32); silu != 0: q, k and v through z sigmoid(z).  o [T][H V] fp32.
+K8S_API int k8s_decay_attn(const void* x, int xs, int dt, int silu, const float* decay, float* state,
+                           const int* seg_row0, const int* seg_pos0, const int* seg_slot, float* o, int n_seg, int H,
+                           int D, int V, hipStream_t s, const int* chunks, int n_chunks, const int* seg_chunk0,
+                           float* cs) {
+  if (n_seg <= 0) return 0;
+  if (H < 1 || D < 1 || V < 1 || (chunks && (n_chunks < 1 || !seg_chunk0 || !cs))) return (int)hipErrorInvalidValue;
+#define K8S_DA(SILU)                                                                                               \
+  K8S_MDT(dt, return (launch_decay_scan<TA, SILU>((const TA*)x, xs, decay, state, seg_row0, seg_pos0, seg_slot, o, \
+                                                  n_seg, H, D, V, s, chunks, n_chunks, seg_chunk0, cs)))
+  if (silu) {
+    K8S_DA(true)
+  }
+  K8S_DA(false)
+#undef K8S_DA
+}
+
+K8S_API int k8s_retention(float* qkvg, int qs, const int* positions, const float* decay, float* state,
+                          const int* seg_row0, const int* seg_pos0, const int* seg_slot, void* out, int n_seg, int H,
+                          int D, int V, int rot, float base, float eps, int odt, hipStream_t s, int T, float* oraw,
+                          const int* chunks, int n_chunks, const int* seg_chunk0, float* cs) {
+  if (n_seg <= 0 || T <= 0) return 0;
+  if (V < 1 || rot < 0 || rot > D || (rot & 1) || (size_t)rot * sizeof(float) > 64 * 1024) return (int)hipErrorInvalidValue;
+  hipLaunchKernelGGL(retention_rope_kernel, dim3(T), dim3(256), rot * sizeof(float) + 8, s, qkvg, qs, positions, H, D,
+                     rot, base);
+  const int rc = launch_decay_scan<float, false>(qkvg, qs, decay, state, seg_row0, seg_pos0, seg_slot, oraw, n_seg, H, D,
+                                                 V, s, chunks, n_chunks, seg_chunk0, cs);
+  if (rc) return rc;
   const int n_rh = T * H;
   K8S_MDT(odt, hipLaunchKernelGGL((head_norm_gate_kernel<TA>), dim3((n_rh + 3) / 4), dim3(256), 0, s, oraw,
                                   qkvg + 2 * H * D + H * V, qs, (TA*)out, n_rh, H, V, eps));

@@ -238,12 +238,17 @@ __global__ void __launch_bounds__(256) postnorm_kernel(float* __restrict__ x, co
 // weight.  The query latent goes to cq [T][QR]; the key-value latent (KR > 0)
 // to the paged latent cache at slots[t] (skipped when negative), and to its
 // transposed twin cache_t when there is one.
+// RD > 0: RD more columns follow, a key part shared by all heads: neighbouring
+// entries 2i, 2i + 1 are turned by the angle whose cosine and sine stand in
+// cs [T][RD] (cos | sin) and go behind the latent in the cache row, padded with
+// zeros to RP numbers (the row is KR + RP wide; the twin holds the latent only).
 template <typename TW, typename TA>
 __global__ void __launch_bounds__(256) latent_norm_kernel(const float* __restrict__ dn, int ld,
                                                           const TW* __restrict__ wq, const TW* __restrict__ wkv,
                                                           const int* __restrict__ slots, TA* __restrict__ cq,
                                                           TA* __restrict__ cache, TA* __restrict__ cache_t, int BS,
-                                                          int QR, int KR, float eps) {
+                                                          int QR, int KR, float eps, int RD, int RP,
+                                                          const float* __restrict__ cs) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const float* row = dn + (size_t)t * ld;
@@ -262,9 +267,40 @@ __global__ void __launch_bounds__(256) latent_norm_kernel(const float* __restric
   const size_t page = slot / BS, off = slot - page * BS;
   for (int c = threadIdx.x; c < KR; c += 256) {
     const float v = row[QR + c] * inv * ldf(wkv, c);
-    stf(cache, (size_t)slot * KR + c, v);
+    stf(cache, (size_t)slot * (KR + RP) + c, v);
     if (cache_t) stf(cache_t, (page * KR + c) * BS + off, v);   // the transposed pages [pages][KR][BS]
   }
+  const int half = RD >> 1;
+  for (int i = threadIdx.x; i < RP; i += 256) {
+    float v = 0.f;
+    if (i < RD) {
+      const float* p = row + QR + KR + (i & ~1);
+      const float co = cs[(size_t)t * RD + (i >> 1)], si = cs[(size_t)t * RD + half + (i >> 1)];
+      v = (i & 1) ? p[1] * co + p[0] * si : p[0] * co - p[1] * si;
+    }
+    stf(cache, (size_t)slot * (KR + RP) + KR + i, v);
+  }
+}
+
+// The last RD entries of every head of q [T][H][N + RD], neighbouring entries turned by the angles of cs [T][RD]
+// (cos | sin), padded with zeros to RP: qr [T][H][RP].
+template <typename TA>
+__global__ void __launch_bounds__(256) rotated_tail_kernel(const TA* __restrict__ q, const float* __restrict__ cs,
+                                                           TA* __restrict__ qr, size_t n, int H, int N, int RD, int RP) {
+  const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;    // a pair of one (row, head)
+  if (e >= n) return;
+  const int hp = RP >> 1, half = RD >> 1;
+  const size_t th = e / hp;
+  const int i = (int)(e - th * hp);
+  float a = 0.f, b = 0.f;
+  if (i < half) {
+    const size_t t = th / H, o = th * (N + RD) + N + 2 * i;
+    const float u = ldf(q, o), v = ldf(q, o + 1), co = cs[t * RD + i], si = cs[t * RD + half + i];
+    a = u * co - v * si;
+    b = v * co + u * si;
+  }
+  stf(qr, th * RP + 2 * i, a);
+  stf(qr, th * RP + 2 * i + 1, b);
 }
 
 }  // namespace k8s
@@ -349,9 +385,24 @@ K8S_API int k8s_postnorm(float* x, const void* y, int y_dt, const void* w, int w
 
 K8S_API int k8s_latent_norm(const float* dn, int ld, const void* wq, const void* wkv, const int* slots, void* cq,
                             void* cache, void* cache_t, int BS, int T, int QR, int KR, float eps, int dt,
-                            hipStream_t s) {
+                            hipStream_t s, int RD, int RP, const float* cs) {
   if (T <= 0) return 0;
+  if (RD < 0 || (RD & 1) || RP < RD || (RP & 1) || (RD && (!cs || KR <= 0))) return (int)hipErrorInvalidValue;
   K8S_DT2(dt, hipLaunchKernelGGL((latent_norm_kernel<TW, TA>), dim3(T), dim3(256), 0, s, dn, ld, (const TW*)wq,
-                                  (const TW*)wkv, slots, (TA*)cq, (TA*)cache, (TA*)cache_t, BS, QR, KR, eps));
+                                  (const TW*)wkv, slots, (TA*)cq, (TA*)cache, (TA*)cache_t, BS, QR, KR, eps,
+                                  RD, RP, cs));
+  return (int)hipGetLastError();
+}
+
+K8S_API int k8s_rotated_tail(const void* q, const float* cs, void* qr, int T, int H, int N, int RD, int RP, int dt,
+                             hipStream_t s) {
+  if (T <= 0 || RP <= 0) return 0;
+  if (H < 1 || N < 0 || RD < 0 || (RD & 1) || (RP & 1) || RP < RD || (RD && !cs)) return (int)hipErrorInvalidValue;
+  const size_t n = (size_t)T * H * (RP / 2);
+  K8S_DT2(dt, {
+    (void)sizeof(TW);
+    hipLaunchKernelGGL((rotated_tail_kernel<TA>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, (const TA*)q, cs,
+                       (TA*)qr, n, H, N, RD, RP);
+  });
   return (int)hipGetLastError();
 }

@@ -169,11 +169,15 @@ class WindowKVPool(KVPool):
     layers may differ in size), plus the values' transposed twin ``vt[i]`` ``[num_blocks, widths[i][1],
     block_size]`` for the layers in ``twins`` (the matrix-core attention kernel's PV operand: 8 consecutive
     keys of one value column contiguous).  With ``twin_only`` those layers hold their values ONLY so
-    (``v[i]`` is None: no kernel of theirs reads token-major values).  A page index means the same token range in every tensor."""
+    (``v[i]`` is None: no kernel of theirs reads token-major values).  The layers in ``in_keys`` read their values out of
+    the key rows (latents: the values are a leading part of every row) and have no token-major values either.  A page
+    index means the same token range in every tensor."""
 
     def __init__(self, widths: List[Tuple[int, int]], num_blocks: int, block_size: int, device,
-                 dtype=torch.bfloat16, twins: Optional[List[bool]] = None, twin_only: bool = False):
+                 dtype=torch.bfloat16, twins: Optional[List[bool]] = None, twin_only: bool = False,
+                 in_keys: Optional[List[bool]] = None):
         self.twin_only = twin_only
+        self.in_keys = list(in_keys) if in_keys is not None else [False] * len(widths)
         self.widths = [(int(a), int(b)) for a, b in widths]
         self.twins = list(twins) if twins is not None else [False] * len(self.widths)
         super().__init__(len(self.widths), 1, 0, num_blocks, block_size, device, dtype)
@@ -183,8 +187,8 @@ class WindowKVPool(KVPool):
         nb, BS = self.num_blocks, self.block_size
         # zero-filled: a stale page never holds a NaN
         self.kc = [torch.zeros(nb, BS, a, dtype=dtype, device=device) for a, _ in self.widths]
-        self.vc = [None if tw and self.twin_only else torch.zeros(nb, BS, b, dtype=dtype, device=device)
-                   for (_, b), tw in zip(self.widths, self.twins)]
+        self.vc = [None if ik or (tw and self.twin_only) else torch.zeros(nb, BS, b, dtype=dtype, device=device)
+                   for (_, b), tw, ik in zip(self.widths, self.twins, self.in_keys)]
         self.vt = [torch.zeros(nb, b, BS, dtype=dtype, device=device) if tw else None
                    for (_, b), tw in zip(self.widths, self.twins)]
 

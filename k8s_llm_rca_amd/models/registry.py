@@ -8,8 +8,9 @@ checkpoint folder's config.json.
 * ``lizesun``             -- :class:`~.lizesun.LizesunModel` (config.json with ``"architecture": "Lizesun"``)
 * ``pumozen``             -- :class:`~.pumozen.PumozenModel` (config.json with ``"architecture": "Pumozen"``)
 * ``sunesun``             -- :class:`~.sunesun.SunesunModel` (config.json with ``"architecture": "Sunesun"``)
+* ``fikerax``             -- :class:`~.fikerax.FikeraxModel` (config.json with ``"architecture": "Fikerax"``)
 
-The last five describe their layers one by one in config.json (``OWN_CONFIG``): their
+The last six describe their layers one by one in config.json (``OWN_CONFIG``): their
 configuration objects are built from it, not from a preset with overrides.
 """
 from __future__ import annotations
@@ -24,7 +25,7 @@ from . import config as C
 # architectures whose config.json lists the layers (``"architecture": <name>``): module, model class
 OWN_CONFIG = {"zasapel": ("zasapel", "ZasapelModel"), "ligipel": ("ligipel", "LigipelModel"),
               "lizesun": ("lizesun", "LizesunModel"), "pumozen": ("pumozen", "PumozenModel"),
-              "sunesun": ("sunesun", "SunesunModel")}
+              "sunesun": ("sunesun", "SunesunModel"), "fikerax": ("fikerax", "FikeraxModel")}
 
 
 def _module(arch: str):

@@ -23,6 +23,7 @@ _err = None
 
 P = ctypes.c_void_p
 I = ctypes.c_int
+L = ctypes.c_long
 F = ctypes.c_float
 
 _SIGS = {
@@ -89,10 +90,11 @@ _SIGS = {
     "k8s_mingru_scan": [P, P, P, P, P, P, P, P, I, I, I, P],
     "k8s_mingru_chunked": [P, P, P, P, P, I, P, P, P, P, P, P, I, I, P],
     "k8s_postnorm": [P, P, I, P, I, P, I, I, F, F, P],
-    "k8s_latent_norm": [P, I, P, P, P, P, P, P, I, I, I, I, F, I, P],
-    "k8s_latent_attn_mfma_ok": [I],
-    "k8s_latent_attn_mfma": [P, P, P, P, I, P, I, P, I, P, P, P, I, I, P, I, I, I, I, F, I, I, P],
-    "k8s_latent_attn_rows": [P, P, P, I, P, P, P, P, I, P, I, I, I, I, I, F, I, P],
+    "k8s_latent_norm": [P, I, P, P, P, P, P, P, I, I, I, I, F, I, P, I, I, P],
+    "k8s_rotated_tail": [P, P, P, I, I, I, I, I, I, P],
+    "k8s_latent_attn_mfma_ok": [I, I],
+    "k8s_latent_attn_mfma": [P, P, P, P, I, P, I, P, I, P, P, P, I, I, P, I, I, I, I, F, I, I, P, L, L, P, I, L, L, I, P],
+    "k8s_latent_attn_rows": [P, P, P, I, P, P, P, P, I, P, I, I, I, I, I, F, I, P, L, L, P, I, L, L, I, P],
     "k8s_polynorm": [P, P, P, I, I, F, I, P],
     "k8s_glu_clamp": [P, P, I, I, F, F, F, I, P],
     "k8s_router": [P, P, I, I, I, I, I, I, P, P, I, P, P, F, I, P, F, I, I],
@@ -108,6 +110,7 @@ _SIGS = {
     "k8s_softcap": [P, ctypes.c_long, F, F, P],
     "k8s_short_conv": [P, I, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, P, P, I],
     "k8s_selective_scan": [P, I, P, P, P, I, I, P, P, P, I, P, P, P, P, P, I, I, I, I, P, P, I, P, P, P],
+    "k8s_decay_attn": [P, I, I, I, P, P, P, P, P, P, I, I, I, I, P, P, I, P, P],
     "k8s_retention": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, F, F, I, P, I, P, P, I, P, P],
     "k8s_window_kv_write": [P, I, I, I, I, P, P, P, I, I, P, P, I],
     "k8s_window_attn_mfma_ok": [I, I, I, I],
@@ -126,7 +129,7 @@ _SIGS = {
     "k8s_matrix_memory": [P, I, P, F, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, P, P, I, P, P, P, P],
     "k8s_head_norm_gate": [P, P, I, P, I, P, I, I, I, F, I, P, P, I, F, F],
     "k8s_ssd_scan": [P, I, P, I, I, P, I, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I, P, P, I, P, P, P],
-    "k8s_hyper_step": [P, P, I, P, P, I, P, P, P, P, F, P, I, I, I, I, P],
+    "k8s_hyper_step": [P, P, I, P, P, I, P, P, P, P, F, P, I, I, I, I, P, P, P, F],
     "k8s_hyper_embed": [P, P, I, F, P, I, P, P, F, P, I, I, I, P],
     "k8s_hyper_read": [P, P, I, I, P, P, F, P, I, I, P],
     "k8s_walks": [P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, P, P, P, P],

@@ -352,13 +352,16 @@ def hyper_embed(ids: torch.Tensor, embed: torch.Tensor, scale: float, x: torch.T
 
 def hyper_step(x: torch.Tensor, y: torch.Tensor, out: torch.Tensor, mix: torch.Tensor, experts: Optional[tuple] = None,
                inn: Optional[torch.Tensor] = None, nw: Optional[torch.Tensor] = None, eps: float = 0.0,
-               out_dtype=None) -> Optional[torch.Tensor]:
+               out_dtype=None, again: Optional[tuple] = None) -> Optional[torch.Tensor]:
     """In place on the streams ``x`` [T, S, W]: ``x_r <- sum_s mix[s, r] x_s + out[r] y`` (all at once from the old ones).
     ``y``: fp32 rows [T, W], or with ``experts = (inv, w)`` the experts' output rows in expert order, joined on the way in
     as ``sum_k w[t, k] y[inv[t K + k]]`` (``inv`` from :func:`..ops.moe.align`, ``w`` [T, K] fp32).  With ``inn, nw`` also
-    returns the next sublayer's input ``rms(sum_s inn[s] x_s) * nw`` of the new streams as activations."""
+    returns the next sublayer's input ``rms(sum_s inn[s] x_s) * nw`` of the new streams as activations.  ``again =
+    (ids, embed, scale)``: the embedding output ``embed[ids] * scale`` is added to every stream as well, in front of that
+    read."""
     T, S, W = x.shape
     read = nw is not None
+    ids, embed, escale = again if again is not None else (None, None, 0.0)
     if use_hip(x):
         assert x.dtype == torch.float32 and x.is_contiguous() and y.is_contiguous() and y.shape[1] == W
         assert out.dtype == mix.dtype == torch.float32 and out.numel() == S and mix.is_contiguous() and mix.numel() == S * S
@@ -371,17 +374,22 @@ def hyper_step(x: torch.Tensor, y: torch.Tensor, out: torch.Tensor, mix: torch.T
         else:
             assert y.dtype == torch.float32 and y.shape[0] == T
         h = None
+        if again is not None:
+            assert read and embed.dtype == out_dtype and embed.is_contiguous() and embed.shape[1] == W
+            assert ids.dtype == torch.int32 and ids.numel() == T
         if read:
             assert inn.dtype == nw.dtype == torch.float32 and inn.numel() == S and nw.numel() == W
             h = torch.empty(T, W, dtype=out_dtype, device=x.device)
         check(lib().k8s_hyper_step(ptr(x), ptr(y), _odt(y.dtype), ptr(inv), ptr(ew), K, ptr(out), ptr(mix), ptr(inn),
-                                   ptr(nw), float(eps), ptr(h), _odt(out_dtype) if read else 1, T, S, W, stream_ptr(x)),
-              "hyper_step")
+                                   ptr(nw), float(eps), ptr(h), _odt(out_dtype) if read else 1, T, S, W, stream_ptr(x),
+                                   ptr(ids), ptr(embed), float(escale)), "hyper_step")
         return h
     if experts is not None:
         inv, ew = experts
         y = (y.float()[inv.long()].view(T, ew.shape[1], W) * ew[:, :, None]).sum(1)
     x.copy_(torch.einsum("sr,tsw->trw", mix, x) + out[None, :, None] * y[:, None])
+    if again is not None:
+        x += (embed[ids.long()].float() * escale)[:, None]
     return _rms_rows(torch.einsum("s,tsw->tw", inn, x), nw, eps, out_dtype) if read else None
 
 

@@ -25,6 +25,7 @@ import torch
 from ._lib import check, lib, ptr, scratch, stream_ptr, use_hip
 
 DECODE_PART = 256   # keys per partition of a decode row (split-KV); borders depend on the key index only
+WINDOW_DECODE_PART = 128   # the same where a window bounds a row's keys
 
 
 @dataclass
@@ -247,30 +248,39 @@ def unit_norm_out(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
 
 def latent_norm(dn: torch.Tensor, wq: torch.Tensor, wkv: Optional[torch.Tensor], slots: torch.Tensor,
                 cache: Optional[torch.Tensor], q_rank: int, kv_rank: int, eps: float, out_dtype,
-                cache_t: Optional[torch.Tensor] = None) -> torch.Tensor:
+                cache_t: Optional[torch.Tensor] = None, tail: int = 0, tail_cs: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Rows of the joint down projection ``dn`` [T, >= q_rank + kv_rank] fp32: the query latent is
     RMS-normed (plain weight) and returned; the key-value latent (``wkv`` given) is RMS-normed and
     written to the paged latent ``cache`` [pages, BS, kv_rank] at ``slots`` (page * BS + offset), and
-    to its transposed twin ``cache_t`` [pages, kv_rank, BS] when given (the MFMA kernels' PV operand)."""
+    to its transposed twin ``cache_t`` [pages, kv_rank, BS] when given (the MFMA kernels' PV operand).
+    ``tail`` > 0: as many further columns of ``dn`` are a key part shared by all heads; its neighbouring entries
+    2i, 2i + 1 are turned by ``tail_cs`` [T, tail] (a :func:`rope_table`) and stand behind the latent in the cache
+    rows [pages, BS, kv_rank + pad], filled up with zeros."""
     T = dn.shape[0]
     cq = torch.empty(T, q_rank, dtype=out_dtype, device=dn.device)
     kr = kv_rank if wkv is not None else 0
+    pad = cache.shape[-1] - kv_rank if kr else 0
     if use_hip(dn):
         assert dn.dtype == torch.float32 and dn.stride(1) == 1 and wq.dtype == out_dtype
-        assert cache is None or (cache.is_contiguous() and cache.dtype == out_dtype and cache.shape[-1] == kv_rank)
+        assert dn.shape[1] >= q_rank + kr + tail and wq.numel() == q_rank
+        assert cache is None or (cache.is_contiguous() and cache.dtype == out_dtype and cache.shape[-1] >= kv_rank + tail)
         ct = cache_t if kr else None
         assert ct is None or (ct.is_contiguous() and ct.dtype == out_dtype and ct.shape[1] == kv_rank)
+        assert not tail or (kr and tail_cs.dtype == torch.float32 and tail_cs.is_contiguous() and tail_cs.shape == (T, tail))
         check(lib().k8s_latent_norm(ptr(dn), dn.stride(0), ptr(wq), ptr(wkv), ptr(slots), ptr(cq), ptr(cache),
                                     ptr(ct), cache.shape[1] if kr else 1, T, q_rank, kr, float(eps),
-                                    _dt(out_dtype), stream_ptr(dn)), "latent_norm")
+                                    _dt(out_dtype), stream_ptr(dn), tail, pad, ptr(tail_cs)), "latent_norm")
         return cq
     q = dn[:, :q_rank]
     cq.copy_((q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * wq.float()).to(out_dtype))
     if kr:
         c = dn[:, q_rank:q_rank + kr]
         c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * wkv.float()
+        row = torch.cat([c, torch.zeros(T, pad)], 1)
+        if tail:
+            row[:, kr:kr + tail] = _turn_pairs(dn[:, q_rank + kr:q_rank + kr + tail], tail_cs)
         ok = slots >= 0
-        cache.view(-1, kr)[slots[ok].long()] = c[ok].to(cache.dtype)
+        cache.view(-1, kr + pad)[slots[ok].long()] = row[ok].to(cache.dtype)
         if cache_t is not None:
             BS = cache.shape[1]
             sl = slots[ok].long()
@@ -278,74 +288,135 @@ def latent_norm(dn: torch.Tensor, wq: torch.Tensor, wkv: Optional[torch.Tensor],
     return cq
 
 
-def mfma_tiles(R: int, dtype, device) -> int:
-    """Query tiles per wave the MFMA attention kernels run prompt portions with for latent rank ``R``
-    (0: they do not take this rank or type -- the vector-pipe kernel runs instead)."""
+def _turn_pairs(x: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
+    """Neighbouring entries of the last dimension turned by the angles of ``cs`` (cos | sin, broadcast over the rest)."""
+    half = cs.shape[-1] // 2
+    co, si = cs[..., :half], cs[..., half:]
+    a, b = x[..., 0::2], x[..., 1::2]
+    return torch.stack([a * co - b * si, b * co + a * si], -1).flatten(-2)
+
+
+def rotated_tail(q: torch.Tensor, cs: torch.Tensor, H: int, N: int, pad: int) -> torch.Tensor:
+    """The entries behind the first ``N`` of every head of ``q`` [T, H (N + R)], neighbours 2i, 2i + 1 turned by ``cs``
+    [T, R] (a :func:`rope_table`), filled up with zeros to ``pad``: [T, H, pad]."""
+    T, R = cs.shape
+    assert q.shape == (T, H * (N + R)) and pad >= R and pad % 2 == 0
+    out = torch.empty(T, H, pad, dtype=q.dtype, device=q.device)
+    if use_hip(q):
+        assert q.is_contiguous() and cs.dtype == torch.float32 and cs.is_contiguous()
+        check(lib().k8s_rotated_tail(ptr(q), ptr(cs), ptr(out), T, H, N, R, pad, _dt(q.dtype), stream_ptr(q)),
+              "rotated_tail")
+        return out
+    out[:, :, :R] = _turn_pairs(q.view(T, H, N + R)[:, :, N:].float(), cs[:, None]).to(q.dtype)
+    out[:, :, R:] = 0
+    return out
+
+
+def mfma_tiles(R: int, dtype, device, tail: int = 0) -> int:
+    """Query tiles per wave the MFMA attention kernels run prompt portions with for latent rank ``R`` and cache rows of
+    ``R + tail`` numbers (0: they do not take these sizes or this type -- the vector-pipe kernel runs instead)."""
     if dtype != torch.bfloat16 or torch.device(device).type != "cuda":
         return 0
-    return int(lib().k8s_latent_attn_mfma_ok(int(R)))
+    return int(lib().k8s_latent_attn_mfma_ok(int(R), int(tail)))
 
 
-def latent_attention_mfma(qa: torch.Tensor, cache: torch.Tensor, cache_t: torch.Tensor, gate: torch.Tensor,
-                          seg: SegMeta, positions: torch.Tensor, scale: float) -> torch.Tensor:
+def _latent_out(qa: torch.Tensor, dtype, head_major: bool) -> torch.Tensor:
+    """[T, H, R], in memory [H][T][R] with ``head_major`` (a batched product over the heads reads it as it is)."""
+    T, H, R = qa.shape
+    if head_major:
+        return torch.empty(H, T, R, dtype=dtype, device=qa.device).transpose(0, 1)
+    return torch.empty(T, H, R, dtype=dtype, device=qa.device)
+
+
+def latent_attention_mfma(qa: torch.Tensor, cache: torch.Tensor, cache_t: torch.Tensor, gate: Optional[torch.Tensor],
+                          seg: SegMeta, positions: torch.Tensor, scale: float, qr: Optional[torch.Tensor] = None,
+                          window: int = 0, sink: Optional[torch.Tensor] = None, head_major: bool = False) -> torch.Tensor:
     """:func:`latent_attention` on the matrix cores: bf16 absorbed queries ``qa`` [T, H, R], the latent
     pages and their transposed twins.  Decode rows (the step's first ``seg.n_single``) are split over
-    partitions of ``DECODE_PART`` keys and merged; prompt portions run one wave per group of tokens."""
+    partitions of keys and merged; prompt portions run one wave per group of tokens."""
     T, H, R = qa.shape
-    BS = cache.shape[1]
-    tiles = mfma_tiles(R, qa.dtype, qa.device)
-    assert tiles and qa.is_contiguous() and cache.is_contiguous() and cache_t.is_contiguous() and BS % 32 == 0
-    assert gate.dtype == torch.float32 and gate.stride(1) == 1 and seg.block_tables.is_contiguous()
-    out = torch.empty(T, H, R, dtype=torch.bfloat16, device=qa.device)
+    BS, W = cache.shape[1], cache.shape[2]
+    tiles = mfma_tiles(R, qa.dtype, qa.device, W - R)
+    assert tiles and qa.stride(2) == 1 and cache.is_contiguous() and cache_t.is_contiguous() and BS % 32 == 0
+    assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[1] >= H)
+    assert cache_t.shape[1:] == (R, BS) and seg.block_tables.is_contiguous() and window >= 0
+    assert (qr is None) == (W == R) and (qr is None or (qr.dtype == qa.dtype and qr.is_contiguous()
+                                                        and qr.shape == (T, H, W - R)))
+    assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H)
+    out = _latent_out(qa, torch.bfloat16, head_major)
     tpi = tiles * (16 // min(H, 16))
     dec, pre, kmax = seg.attn_items(tpi)
     L, st = lib(), stream_ptr(qa)
     bt, maxb = seg.block_tables, seg.block_tables.shape[1]
+    gs = gate.stride(0) if gate is not None else 0
+    more = (qa.stride(0), qa.stride(1), ptr(qr), W - R, out.stride(0), out.stride(1), int(window), ptr(sink))
     if dec.shape[0]:
-        n_parts = -(-kmax // DECODE_PART)
+        part = DECODE_PART
+        n_parts = -(-kmax // part)
+        if window > 0:      # a row's parts start at the one its first visible key lies in
+            part = WINDOW_DECODE_PART
+            n_parts = min(-(-kmax // part), (min(int(window), kmax) + part - 2) // part + 1)
         nd = seg.n_single
         part_o = scratch(nd * H * n_parts * R, torch.float32, qa.device)
         part_ml = scratch(nd * H * n_parts * 2, torch.float32, qa.device)
         check(L.k8s_latent_attn_mfma(ptr(qa), ptr(cache), ptr(cache_t), ptr(bt), maxb, ptr(dec), dec.shape[0],
-                                     ptr(gate), gate.stride(0), ptr(out), ptr(part_o), ptr(part_ml), n_parts,
-                                     DECODE_PART, ptr(positions), nd, H, R, BS, float(scale), 1, 1, st),
+                                     ptr(gate), gs, ptr(out), ptr(part_o), ptr(part_ml), n_parts,
+                                     part, ptr(positions), nd, H, R, BS, float(scale), 1, 1, st, *more),
               "latent_attn_mfma (decode)")
     if pre.shape[0]:
         check(L.k8s_latent_attn_mfma(ptr(qa), ptr(cache), ptr(cache_t), ptr(bt), maxb, ptr(pre), pre.shape[0],
-                                     ptr(gate), gate.stride(0), ptr(out), None, None, 1, DECODE_PART, None, 0,
-                                     H, R, BS, float(scale), 0, tiles, st), "latent_attn_mfma (prefill)")
+                                     ptr(gate), gs, ptr(out), None, None, 1, DECODE_PART, None, 0,
+                                     H, R, BS, float(scale), 0, tiles, st, *more), "latent_attn_mfma (prefill)")
     return out
 
 
-def latent_attention(qa: torch.Tensor, cache: torch.Tensor, gate: torch.Tensor, seg: SegMeta, scale: float,
-                     out_dtype) -> torch.Tensor:
+def latent_attention(qa: torch.Tensor, cache: torch.Tensor, gate: Optional[torch.Tensor], seg: SegMeta, scale: float,
+                     out_dtype, qr: Optional[torch.Tensor] = None, window: int = 0, sink: Optional[torch.Tensor] = None,
+                     head_major: bool = False) -> torch.Tensor:
     """Causal attention of absorbed queries ``qa`` [T, H, R] fp32 over the paged latents ``cache``
     [pages, BS, R]: ``p = softmax(scale * qa . c_j)`` over the keys up to the row's own position,
-    output ``sigmoid(gate[t, h]) * sum_j p_j c_j`` [T, H, R] (``gate`` fp32, row stride free)."""
+    output ``sigmoid(gate[t, h]) * sum_j p_j c_j`` [T, H, R] (``gate`` fp32, row stride free; None: no gate).
+    ``qr`` [T, H, P] fp32: the cache rows are [R + P], a key part shared by the heads behind the latent, and
+    ``qr . k_j`` is added to the product.  ``window`` > 0: position i sees j with ``i - j < window``.  ``sink`` [H]
+    fp32: ``exp(sink_h)`` is added to head h's denominator.  ``head_major``: the result lies [H][T][R] in memory."""
     T, H, R = qa.shape
-    BS = cache.shape[1]
-    out = torch.empty(T, H, R, dtype=out_dtype, device=qa.device)
+    BS, W = cache.shape[1], cache.shape[2]
+    assert (qr is None) == (W == R)
+    out = _latent_out(qa, out_dtype, head_major)
     if use_hip(qa):
-        assert qa.dtype == torch.float32 and qa.is_contiguous() and cache.is_contiguous() and cache.dtype == out_dtype
-        assert gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[1] >= H
+        assert qa.dtype == torch.float32 and qa.stride(2) == 1 and cache.is_contiguous() and cache.dtype == out_dtype
+        assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[1] >= H)
+        assert qr is None or (qr.dtype == torch.float32 and qr.is_contiguous() and qr.shape == (T, H, W - R))
+        assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H)
         assert seg.block_tables.is_contiguous()
         check(lib().k8s_latent_attn_rows(ptr(qa), ptr(cache), ptr(seg.block_tables), seg.block_tables.shape[1],
                                          ptr(seg.row_seg), ptr(seg.seg_row0), ptr(seg.seg_pos0), ptr(gate),
-                                         gate.stride(0), ptr(out), 0, T, H, R, BS, float(scale), _dt(out_dtype),
-                                         stream_ptr(qa)), "latent_attn_rows")
+                                         gate.stride(0) if gate is not None else 0, ptr(out), 0, T, H, R, BS,
+                                         float(scale), _dt(out_dtype), stream_ptr(qa), qa.stride(0), qa.stride(1),
+                                         ptr(qr), W - R, out.stride(0), out.stride(1), int(window), ptr(sink)),
+              "latent_attn_rows")
         return out
-    flat = cache.view(-1, R)
+    flat = cache.view(-1, W)
     for s in range(seg.n_seg):
         a, b, p0 = seg.row0_host[s], seg.row0_host[s + 1], seg.pos0_host[s]
         n_ctx = p0 + b - a
         pages = seg.block_tables[s].long()
         kp = torch.arange(n_ctx)
-        c = flat[pages[kp // BS] * BS + kp % BS].float()                      # [ctx, R]
-        sc = torch.einsum("thr,jr->thj", qa[a:b], c) * scale
-        vis = kp[None, :] <= (p0 + torch.arange(b - a))[:, None]
-        sc = sc.masked_fill(~vis[:, None, :], float("-inf"))
-        o = torch.einsum("thj,jr->thr", torch.softmax(sc, -1), c)
-        out[a:b] = (o * torch.sigmoid(gate[a:b, :H])[:, :, None]).to(out_dtype)
+        c = flat[pages[kp // BS] * BS + kp % BS].float()                      # [ctx, R (+ P)]
+        sc = torch.einsum("thr,jr->thj", qa[a:b].float(), c[:, :R])
+        if qr is not None:
+            sc = sc + torch.einsum("thr,jr->thj", qr[a:b].float(), c[:, R:])
+        dist = (p0 + torch.arange(b - a))[:, None] - kp[None, :]
+        vis = dist >= 0
+        if window > 0:
+            vis &= dist < window
+        sc = (sc * scale).masked_fill(~vis[:, None, :], float("-inf"))
+        if sink is not None:                                                   # one more score without a value
+            p = torch.softmax(torch.cat([sc, sink.view(1, H, 1).expand(b - a, H, 1)], -1), -1)[..., :-1]
+        else:
+            p = torch.softmax(sc, -1)
+        o = torch.einsum("thj,jr->thr", p, c[:, :R])
+        out[a:b] = (o if gate is None else o * torch.sigmoid(gate[a:b, :H])[:, :, None]).to(out_dtype)
     return out
 
 
@@ -540,6 +611,42 @@ def retention(qkvg: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor, r
     return out
 
 
+def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor, state: torch.Tensor, seg: SegMeta,
+                    silu: bool = False) -> torch.Tensor:
+    """Linear attention with a fixed decay per head, fp32: rows of ``x`` [T, >= 2 H D + H V] = (q | k | v) activations
+    (row stride free), with ``silu`` each of them through ``z sigmoid(z)`` first;  ``S <- decay_h S + k v^T``;  ``o = S^T q``.
+    ``decay`` [H] fp32.  ``state`` [slots, H, D, V] fp32 is read (past position 0) and advanced.  Returns o [T, H V] fp32."""
+    T = x.shape[0]
+    out = torch.empty(T, H * V, dtype=torch.float32, device=x.device)
+    if use_hip(x):
+        assert x.stride(1) == 1 and x.shape[1] >= H * (2 * D + V) and decay.dtype == torch.float32 and decay.numel() == H
+        assert state.is_contiguous() and state.dtype == torch.float32 and state.shape[1:] == (H, D, V)
+        # long portions: chunks in parallel (end states from zero, a carry over the chunks, the chunks
+        # again from their start states); short ones token by token
+        cr = seg.chunk_ranges(SSM_CHUNK, 2 * SSM_CHUNK) if seg.n_seg * H * V * 8 < SEQ_FILL_LANES else None
+        chunks, c0, cs, nch = None, None, None, 0
+        if cr is not None:
+            chunks, c0 = cr
+            nch = chunks.shape[0]
+            cs = scratch(nch * H * D * V, torch.float32, x.device)
+        check(lib().k8s_decay_attn(ptr(x), x.stride(0), _dt(x.dtype), int(silu), ptr(decay), ptr(state),
+                                   ptr(seg.seg_row0), ptr(seg.seg_pos0), ptr(seg.seg_slot), ptr(out), seg.n_seg, H, D, V,
+                                   stream_ptr(x), ptr(chunks), nch, ptr(c0), ptr(cs)), "decay_attn")
+        return out
+    qkv = x[:, :H * (2 * D + V)].float()
+    if silu:
+        qkv = torch.nn.functional.silu(qkv)
+    q, k, v = qkv[:, :H * D].view(T, H, D), qkv[:, H * D:2 * H * D].view(T, H, D), qkv[:, 2 * H * D:].view(T, H, V)
+    for s in range(seg.n_seg):
+        a, e, p0, sl = seg.row0_host[s], seg.row0_host[s + 1], seg.pos0_host[s], seg.slot_host[s]
+        S = state[sl].clone() if p0 > 0 else torch.zeros(H, D, V)
+        for r in range(a, e):
+            S = decay[:, None, None] * S + k[r][:, :, None] * v[r][:, None, :]
+            out[r] = torch.einsum("hdv,hd->hv", S, q[r]).reshape(-1)
+        state[sl] = S
+    return out
+
+
 def window_mfma_ok(H: int, G: int, D: int, V: int, dtype, device) -> bool:
     """Whether the matrix-core window attention kernel takes these sizes (bf16 on the device only;
     the vector-pipe kernel runs everything else)."""
@@ -655,12 +762,14 @@ class Rope:
     pairs: bool = False
 
 
-def make_rope(dims: int, base: float, device, pairs: bool = False, yarn: Optional[Tuple[float, float, float, float]] = None
-              ) -> Rope:
+def make_rope(dims: int, base: float, device, pairs: bool = False, yarn: Optional[Tuple[float, float, float, float]] = None,
+              stretch: Optional[Tuple[float, float, float, float]] = None) -> Rope:
     """:class:`Rope` with ``freq[i] = base^(-2 i / dims)``.  ``yarn = (factor, original, fast, slow)``: a pair that turns
     more than ``fast`` times within ``original`` positions keeps its frequency, one that turns less than ``slow`` times
     has it divided by ``factor``, with a linear ramp over the pair index between the two, and
-    ``amp = 0.1 ln(factor) + 1``."""
+    ``amp = 0.1 ln(factor) + 1``.  ``stretch = (factor, low, high, original)``: by wavelength ``l = 2 pi / freq`` -- kept
+    below ``original / high``, divided by ``factor`` above ``original / low``, and between the two a mix of both by
+    ``s = (original / l - low) / (high - low)``, the kept one's share."""
     f = torch.tensor([base ** (-2.0 * i / dims) for i in range(dims // 2)], dtype=torch.float64)
     amp = 1.0
     if yarn is not None:
@@ -673,6 +782,11 @@ def make_rope(dims: int, base: float, device, pairs: bool = False, yarn: Optiona
         ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
         f = f / factor * ramp + f * (1.0 - ramp)
         amp = 0.1 * math.log(factor) + 1.0
+    if stretch is not None:
+        factor, low, high, original = (float(v) for v in stretch)
+        turns = original * f / (2.0 * math.pi)                     # original / wavelength
+        s = ((turns - low) / (high - low) if high != low else torch.zeros_like(turns))
+        f = torch.where(turns > high, f, torch.where(turns < low, f / factor, (1.0 - s) * f / factor + s * f))
     return Rope(dims, f.to(device), amp, pairs)
 
 
