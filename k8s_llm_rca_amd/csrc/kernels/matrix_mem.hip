@@ -396,8 +396,9 @@ __global__ void __launch_bounds__(256) delta_carry_kernel(MatArgs p, const int* 
 // optional): one wave per (row, head).  w and gate are optional (absent: 1).
 // w is indexed h * wh + c: wh = V for a weight of all heads' size, 0 for one shared by the heads.
 // sub: o holds two results per head, [r][h][2][V], and u = o[.][0] - lam o[.][1] (two score maps joined).
-template <typename TA>
-__global__ void __launch_bounds__(256) head_norm_sigmoid_kernel(const float* __restrict__ o, const float* __restrict__ gate,
+// gate (TG) is fp32 or an activation.
+template <typename TA, typename TG>
+__global__ void __launch_bounds__(256) head_norm_sigmoid_kernel(const float* __restrict__ o, const TG* __restrict__ gate,
                                                                 int gs, const float* __restrict__ w, int wh,
                                                                 TA* __restrict__ out, int n_rh, int H, int V, float eps,
                                                                 const float* __restrict__ mul, int sub, float lam,
@@ -413,12 +414,69 @@ __global__ void __launch_bounds__(256) head_norm_sigmoid_kernel(const float* __r
     ss = fmaf(u, u, ss);
   }
   const float rn = mu * oscale / sqrtf(wave_sum(ss) / (float)V + eps);
-  const float* g = gate ? gate + (size_t)r * gs + (size_t)h * V : nullptr;
+  const TG* g = gate ? gate + (size_t)r * gs + (size_t)h * V : nullptr;
   const float* wp = w ? w + (size_t)h * wh : nullptr;
   for (int c = lane; c < V; c += 64) {
     const float u = sub ? op[c] - lam * op[V + c] : op[c];
-    stx(out, (size_t)rh * V + c, u * rn * (wp ? wp[c] : 1.f) * (g ? sigmoid_f(g[c]) : 1.f));
+    stx(out, (size_t)rh * V + c, u * rn * (wp ? wp[c] : 1.f) * (g ? sigmoid_f(ldx(g, c)) : 1.f));
   }
+}
+
+// The same with one norm over a whole row of V (a multiple of 4): a workgroup per row, four neighbouring entries per
+// thread and round, the row in registers between the sum of squares and the output.
+constexpr int kRowRounds = 4;
+template <typename TA, typename TG>
+__global__ void __launch_bounds__(1024) row_norm_sigmoid_kernel(const float* __restrict__ o, const TG* __restrict__ gate,
+                                                                int gs, const float* __restrict__ w,
+                                                                TA* __restrict__ out, int V, float eps) {
+  __shared__ float red[16];
+  const size_t row = (size_t)blockIdx.x * V;
+  const int step = 4 * blockDim.x;
+  f32x4 v[kRowRounds];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < kRowRounds; ++k) {
+    const int c = 4 * threadIdx.x + k * step;
+    if (c < V) {
+      v[k] = *reinterpret_cast<const f32x4*>(o + row + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) ss = fmaf(v[k][i], v[k][i], ss);
+    }
+  }
+  const float rn = 1.f / sqrtf(block_sum(ss, red) / (float)V + eps);
+#pragma unroll
+  for (int k = 0; k < kRowRounds; ++k) {
+    const int c = 4 * threadIdx.x + k * step;
+    if (c < V) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float u = v[k][i] * rn;
+        if (w) u *= w[c + i];
+        if (gate) u *= 1.f / (1.f + __expf(-ldx(gate, (size_t)blockIdx.x * gs + c + i)));
+        v[k][i] = u;
+      }
+      if constexpr (sizeof(TA) == 4)
+        *reinterpret_cast<f32x4*>(out + row + c) = v[k];
+      else
+        *reinterpret_cast<u16x4*>(out + row + c) = u16x4{f2bf(v[k][0]), f2bf(v[k][1]), f2bf(v[k][2]), f2bf(v[k][3])};
+    }
+  }
+}
+
+template <typename TA, typename TG>
+static int launch_head_norm(const float* o, const void* gate, int gs, const float* w, int wh, void* out, int T, int H,
+                            int V, float eps, hipStream_t s, const float* mul, int sub, float lam, float oscale) {
+  const int n_rh = T * H;
+  if (H == 1 && !mul && !sub && oscale == 1.f && V % 4 == 0 && V >= 256 && V <= 4 * 1024 * kRowRounds &&
+      (((uintptr_t)o | (uintptr_t)out) & 15) == 0) {
+    const int want = (V / 4 + 63) / 64 * 64;
+    hipLaunchKernelGGL((row_norm_sigmoid_kernel<TA, TG>), dim3(T), dim3(want > 1024 ? 1024 : want), 0, s, o,
+                       (const TG*)gate, gs, w, (TA*)out, V, eps);
+  } else {
+    hipLaunchKernelGGL((head_norm_sigmoid_kernel<TA, TG>), dim3((n_rh + 3) / 4), dim3(256), 0, s, o, (const TG*)gate, gs,
+                       w, wh, (TA*)out, n_rh, H, V, eps, mul, sub, lam, oscale);
+  }
+  return (int)hipGetLastError();
 }
 
 template <int DPT, int KIND, int MODE, bool FULL, typename TA>
@@ -548,17 +606,15 @@ K8S_API int k8s_matrix_memory(const float* x, int xs, const float* gate_bias, fl
   return (int)hipGetLastError();
 }
 
-// mul (optional) [T][H]: o is multiplied by it before the norm
-K8S_API int k8s_head_norm_gate(const float* o, const float* gate, int gs, const float* w, int wh, void* out, int T,
+// mul (optional) [T][H]: o is multiplied by it before the norm.  odt / gdt: the types of out and gate (0 bf16, 1 fp32)
+K8S_API int k8s_head_norm_gate(const float* o, const void* gate, int gs, const float* w, int wh, void* out, int T,
                                int H, int V, float eps, int odt, hipStream_t s, const float* mul, int sub, float lam,
-                               float oscale) {
+                               float oscale, int gdt) {
   if (T <= 0) return 0;
-  const int n_rh = T * H;
-  if (odt == 0)
-    hipLaunchKernelGGL((head_norm_sigmoid_kernel<uint16_t>), dim3((n_rh + 3) / 4), dim3(256), 0, s, o, gate, gs, w, wh,
-                       (uint16_t*)out, n_rh, H, V, eps, mul, sub, lam, oscale);
-  else
-    hipLaunchKernelGGL((head_norm_sigmoid_kernel<float>), dim3((n_rh + 3) / 4), dim3(256), 0, s, o, gate, gs, w, wh,
-                       (float*)out, n_rh, H, V, eps, mul, sub, lam, oscale);
-  return (int)hipGetLastError();
+#define K8S_HN(TA, TG) return launch_head_norm<TA, TG>(o, gate, gs, w, wh, out, T, H, V, eps, s, mul, sub, lam, oscale)
+  if (odt == 0 && gdt == 0) K8S_HN(uint16_t, uint16_t);
+  if (odt == 0) K8S_HN(uint16_t, float);
+  if (gdt == 0) K8S_HN(float, uint16_t);
+  K8S_HN(float, float);
+#undef K8S_HN
 }

@@ -377,7 +377,7 @@ class FikeraxModel:
     def _lightning(self, i: int, h: torch.Tensor, inp: S.SegStepInputs, state: torch.Tensor) -> torch.Tensor:
         L, c = self.layers[i], self.cfg.layers[i].mix
         HV = c.heads * c.vdim
-        x = proj_f32out(h, L["w_in"])
+        x = linear(h, L["w_in"])                                             # q | k | v | gate as activations
         o = S.decay_attention(x, c.heads, c.dim, c.vdim, L["decay"], state, inp.seg, silu=True)
         y = S.head_norm_gate(o, x[:, x.shape[1] - HV:], L["mem_norm"], 1, HV, self.cfg.norm_eps, self.dtype)
         return proj_f32out(y, L["wo"])

@@ -111,6 +111,8 @@ _SIGS = {
     "k8s_short_conv": [P, I, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, P, P, I],
     "k8s_selective_scan": [P, I, P, P, P, I, I, P, P, P, I, P, P, P, P, P, I, I, I, I, P, P, I, P, P, P],
     "k8s_decay_attn": [P, I, I, I, P, P, P, P, P, P, I, I, I, I, P, P, I, P, P],
+    "k8s_decay_attn_mfma_ok": [I, I],
+    "k8s_decay_attn_mfma": [P, I, I, P, P, P, P, P, P, I, I, I, I, P, P, I, P, P],
     "k8s_retention": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, F, F, I, P, I, P, P, I, P, P],
     "k8s_window_kv_write": [P, I, I, I, I, P, P, P, I, I, P, P, I],
     "k8s_window_attn_mfma_ok": [I, I, I, I],
@@ -127,7 +129,7 @@ _SIGS = {
     "k8s_masked_attn_mfma": [P, P, P, P, I, P, I, P, P, I, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, P, I, I],
     "k8s_gated_delta": [P, I, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, F, P, P, I, P, P, P],
     "k8s_matrix_memory": [P, I, P, F, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, P, P, I, P, P, P, P],
-    "k8s_head_norm_gate": [P, P, I, P, I, P, I, I, I, F, I, P, P, I, F, F],
+    "k8s_head_norm_gate": [P, P, I, P, I, P, I, I, I, F, I, P, P, I, F, F, I],
     "k8s_ssd_scan": [P, I, P, I, I, P, I, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I, P, P, I, P, P, P],
     "k8s_hyper_step": [P, P, I, P, P, I, P, P, P, P, F, P, I, I, I, I, P, P, P, F],
     "k8s_hyper_embed": [P, P, I, F, P, I, P, P, F, P, I, I, I, P],

@@ -4,7 +4,8 @@ minGRU recurrence, the post-sublayer norm of an fp32 residual, attention over a
 paged latent cache (``csrc/kernels/seq_ops.hip``, ``latent_attn.hip``), window
 attention and recurrent mixers (``mixer_ops.hip``, ``window_attn.hip``), masked
 softmax attention behind a q / k preparation pass and matrix-state recurrences
-(``masked_attn.hip``, ``matrix_mem.hip``).
+(``masked_attn.hip``, ``matrix_mem.hip``), linear attention on the matrix cores
+(``linear_attn.hip``).
 
 A step's rows come in SEGMENTS (:class:`SegMeta`): consecutive rows of one
 sequence -- a decode token or a portion of a prompt.  Device tensors run the HIP
@@ -622,13 +623,24 @@ def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor
         assert x.stride(1) == 1 and x.shape[1] >= H * (2 * D + V) and decay.dtype == torch.float32 and decay.numel() == H
         assert state.is_contiguous() and state.dtype == torch.float32 and state.shape[1:] == (H, D, V)
         # long portions: chunks in parallel (end states from zero, a carry over the chunks, the chunks
-        # again from their start states); short ones token by token
-        cr = seg.chunk_ranges(SSM_CHUNK, 2 * SSM_CHUNK) if seg.n_seg * H * V * 8 < SEQ_FILL_LANES else None
+        # again from their start states); short ones token by token.  On the matrix cores a portion goes in
+        # blocks of 64 tokens, and its chunks are ranges of several blocks
+        longest = max(b - a for a, b in zip(seg.row0_host[:-1], seg.row0_host[1:]))
+        mfma = longest >= LIN_MFMA_ROWS and decay_mfma_ok(D, V, x.dtype, x.device) and x.stride(0) % 4 == 0
+        if mfma:
+            cr = seg.chunk_ranges(LIN_CHUNK, LIN_CHUNK) if seg.n_seg * H * -(-V // 128) < LIN_FILL_GROUPS else None
+        else:
+            cr = seg.chunk_ranges(SSM_CHUNK, 2 * SSM_CHUNK) if seg.n_seg * H * V * 8 < SEQ_FILL_LANES else None
         chunks, c0, cs, nch = None, None, None, 0
         if cr is not None:
             chunks, c0 = cr
             nch = chunks.shape[0]
             cs = scratch(nch * H * D * V, torch.float32, x.device)
+        if mfma:
+            check(lib().k8s_decay_attn_mfma(ptr(x), x.stride(0), int(silu), ptr(decay), ptr(state), ptr(seg.seg_row0),
+                                            ptr(seg.seg_pos0), ptr(seg.seg_slot), ptr(out), seg.n_seg, H, D, V,
+                                            stream_ptr(x), ptr(chunks), nch, ptr(c0), ptr(cs)), "decay_attn_mfma")
+            return out
         check(lib().k8s_decay_attn(ptr(x), x.stride(0), _dt(x.dtype), int(silu), ptr(decay), ptr(state),
                                    ptr(seg.seg_row0), ptr(seg.seg_pos0), ptr(seg.seg_slot), ptr(out), seg.n_seg, H, D, V,
                                    stream_ptr(x), ptr(chunks), nch, ptr(c0), ptr(cs)), "decay_attn")
@@ -645,6 +657,18 @@ def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor
             out[r] = torch.einsum("hdv,hd->hv", S, q[r]).reshape(-1)
         state[sl] = S
     return out
+
+
+LIN_MFMA_ROWS = 17      # rows of a step's longest portion from which the matrix-core form runs
+LIN_CHUNK = 128         # rows per range where ranges of a portion run in parallel
+LIN_FILL_GROUPS = 128   # workgroups (segments x heads x 128 value columns) from which whole portions fill the chip
+
+
+def decay_mfma_ok(D: int, V: int, dtype, device) -> bool:
+    """Whether the matrix-core form of :func:`decay_attention` takes these sizes (bf16 on the device only)."""
+    if dtype != torch.bfloat16 or torch.device(device).type != "cuda":
+        return False
+    return bool(lib().k8s_decay_attn_mfma_ok(int(D), int(V)))
 
 
 def window_mfma_ok(H: int, G: int, D: int, V: int, dtype, device) -> bool:
@@ -1027,21 +1051,23 @@ def head_norm_gate(o: torch.Tensor, gate: Optional[torch.Tensor], w: Optional[to
                    out_dtype, mul: Optional[torch.Tensor] = None, sub_lambda: Optional[float] = None,
                    out_scale: float = 1.0) -> torch.Tensor:
     """``u / rms(u over each head's V) * w * sigmoid(gate) * out_scale`` of fp32 rows ``o`` [T, H V], ``u = o * mul`` with
-    ``mul`` [T, H] where given; ``w`` [V] (shared by the heads) or [H V] or None; ``gate`` [T, H V] fp32 (row stride
-    free) or None.  With ``sub_lambda`` the rows hold two results per head, [T, H, 2, V], and
+    ``mul`` [T, H] where given; ``w`` [V] (shared by the heads) or [H V] or None; ``gate`` [T, H V] fp32 or bf16 (row
+    stride free) or None.  With ``sub_lambda`` the rows hold two results per head, [T, H, 2, V], and
     ``u = o[:, :, 0] - sub_lambda * o[:, :, 1]`` (two score maps over the same values, joined)."""
     T = o.shape[0]
     out = torch.empty(T, H * V, dtype=out_dtype, device=o.device)
     sub = sub_lambda is not None
     if use_hip(o):
         assert o.dtype == torch.float32 and o.is_contiguous() and o.shape[1] == H * V * (2 if sub else 1)
-        assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[1] >= H * V)
+        assert gate is None or (gate.dtype in (torch.float32, torch.bfloat16) and gate.stride(1) == 1
+                                and gate.shape[1] >= H * V)
         assert w is None or (w.dtype == torch.float32 and w.numel() in (V, H * V))
         assert mul is None or (mul.dtype == torch.float32 and mul.is_contiguous() and mul.numel() == T * H)
         check(lib().k8s_head_norm_gate(ptr(o), ptr(gate), gate.stride(0) if gate is not None else 0, ptr(w),
                                        V if w is not None and w.numel() == H * V else 0,
                                        ptr(out), T, H, V, float(eps), _dt(out_dtype), stream_ptr(o), ptr(mul),
-                                       int(sub), float(sub_lambda or 0.0), float(out_scale)), "head_norm_gate")
+                                       int(sub), float(sub_lambda or 0.0), float(out_scale),
+                                       _dt(gate.dtype) if gate is not None else 1), "head_norm_gate")
         return out
     if sub:
         oh = o.view(T, H, 2, V)
@@ -1054,7 +1080,7 @@ def head_norm_gate(o: torch.Tensor, gate: Optional[torch.Tensor], w: Optional[to
     if w is not None:
         oh = oh * (w.view(H, V) if w.numel() == H * V else w.view(1, V))
     if gate is not None:
-        oh = oh * torch.sigmoid(gate[:, :H * V]).view(T, H, V)
+        oh = oh * torch.sigmoid(gate[:, :H * V].float()).view(T, H, V)
     out.copy_(oh.reshape(T, H * V).to(out_dtype))
     return out
 
