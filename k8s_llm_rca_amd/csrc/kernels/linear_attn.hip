@@ -41,8 +41,6 @@ struct LinArgs {
   int H, V;
 };
 
-__device__ __forceinline__ float silu_hw(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
-
 // dec^n by repeated squaring
 __device__ __forceinline__ float ipow(float dec, int n) {
   float r = 1.f, b = dec;

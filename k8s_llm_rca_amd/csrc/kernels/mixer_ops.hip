@@ -417,7 +417,14 @@ __global__ void __launch_bounds__(256) retention_rope_kernel(float* __restrict__
 }
 
 // The scan of step 2 by itself is linear attention with one decay per head (k8s_decay_attn): rows of x (TA,
-// stride xs) = q [H][D] | k [H][D] | v [H][V], with SILU each of them through z sigmoid(z) first.
+// stride xs) = q [H][D] | k [H][D] | v [H][V], with SILU each of them through z sigmoid(z), as an activation of type
+// TA, first (the matrix-core form in linear_attn.hip has the same operands).
+template <typename TA>
+__device__ __forceinline__ float act_silu(float z);
+template <>
+__device__ __forceinline__ float act_silu<float>(float z) { return silu_f(z); }
+template <>
+__device__ __forceinline__ float act_silu<uint16_t>(float z) { return bf2f(f2bf(silu_hw(z))); }
 constexpr int kRetTb = 16;    // tokens per batch
 // MODE 0: blockIdx.x = segment, from the slot's state (or zero at position 0) to the slot's state.
 // Long segments are cut into chunks ([n][4]: segment, first row, rows, -) that run in parallel:
@@ -469,13 +476,13 @@ __global__ void __launch_bounds__(256) retention_scan_kernel(const TA* __restric
       const int tb = e / D, d = e - tb * D;
       const size_t row = (size_t)(t0 + tb) * qs;
       const float qv = ldm(qkvg, row + hh * D + d), kv = ldm(qkvg, row + (H + hh) * D + d);
-      sq[e] = SILU ? DecayExp<TA>::silu(qv) : qv;
-      sk[e] = SILU ? DecayExp<TA>::silu(kv) : kv;
+      sq[e] = SILU ? act_silu<TA>(qv) : qv;
+      sk[e] = SILU ? act_silu<TA>(kv) : kv;
     }
     for (int e = tid; e < nb * VBS; e += 256) {
       const int tb = e / VBS, vv = e - tb * VBS;
       const float xv = v0 + vv < V ? ldm(qkvg, (size_t)(t0 + tb) * qs + 2 * H * D + hh * V + v0 + vv) : 0.f;
-      sv[e] = SILU ? DecayExp<TA>::silu(xv) : xv;
+      sv[e] = SILU ? act_silu<TA>(xv) : xv;
     }
     __syncthreads();
     if (dg < NDG) {

@@ -615,7 +615,7 @@ def retention(qkvg: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor, r
 def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor, state: torch.Tensor, seg: SegMeta,
                     silu: bool = False) -> torch.Tensor:
     """Linear attention with a fixed decay per head, fp32: rows of ``x`` [T, >= 2 H D + H V] = (q | k | v) activations
-    (row stride free), with ``silu`` each of them through ``z sigmoid(z)`` first;  ``S <- decay_h S + k v^T``;  ``o = S^T q``.
+    (row stride free), with ``silu`` each of them through ``z sigmoid(z)`` first, as activations of ``x``'s type;  ``S <- decay_h S + k v^T``;  ``o = S^T q``.
     ``decay`` [H] fp32.  ``state`` [slots, H, D, V] fp32 is read (past position 0) and advanced.  Returns o [T, H V] fp32."""
     T = x.shape[0]
     out = torch.empty(T, H * V, dtype=torch.float32, device=x.device)
@@ -647,7 +647,7 @@ def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor
         return out
     qkv = x[:, :H * (2 * D + V)].float()
     if silu:
-        qkv = torch.nn.functional.silu(qkv)
+        qkv = torch.nn.functional.silu(qkv).to(x.dtype).float()
     q, k, v = qkv[:, :H * D].view(T, H, D), qkv[:, H * D:2 * H * D].view(T, H, D), qkv[:, 2 * H * D:].view(T, H, V)
     for s in range(seg.n_seg):
         a, e, p0, sl = seg.row0_host[s], seg.row0_host[s + 1], seg.pos0_host[s], seg.slot_host[s]
