@@ -53,7 +53,7 @@ __device__ __forceinline__ float relu_sq_f(float v) {
 
 // z sigmoid(z) with the hardware exponential, for results that become bf16: every kernel that rounds it to bf16 uses this
 // one, so the prompt and the decode form of a layer hold the same activations.
-__device__ __forceinline__ float silu_hw(float z) { return __fdividef(z, 1.f + __expf(-z)); }
+__device__ __forceinline__ float silu_hw(float z) { return z * __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
 
 // RoPE of one (x[i], x[i + 64]) pair in a fixed operation order -- no choice
 // left to the compiler's contraction -- so every kernel that rotates (rope_kv,

@@ -184,6 +184,43 @@ __device__ __forceinline__ void sta4<uint16_t>(uint16_t* p, size_t i, const f32x
   *reinterpret_cast<u16x4*>(p + i) = u16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])};
 }
 
+// The value columns of TR rows from r0 (nr of them exist) to their pages: row-major, and a column of TR rows whose slots
+// are TR aligned neighbours of one page to the transposed page in one store.
+template <typename TA, int TR>
+__device__ __forceinline__ void write_values(const float* __restrict__ x, int qs, int r0, int nr, int NV, int v_col,
+                                             const float* __restrict__ bias, const int* __restrict__ slots,
+                                             TA* __restrict__ vc, TA* __restrict__ vt, int BS, int tid) {
+  if (NV == 0) return;
+  const int s0 = slots[r0];
+  bool run = TR > 1 && nr == TR && s0 >= 0 && s0 % TR == 0 && BS % TR == 0;    // then a page holds all TR
+  for (int k = 1; k < nr; ++k) run = run && slots[r0 + k] == s0 + k;
+  for (int c = tid; c < NV; c += 256) {
+    const float vb = bias ? bias[v_col + c] : 0.f;
+    float v[TR];
+#pragma unroll
+    for (int k = 0; k < TR; ++k) v[k] = k < nr ? x[(size_t)(r0 + k) * qs + v_col + c] + vb : 0.f;
+    if (vt && run) {
+      const int page = s0 / BS;
+      TA* o = vt + ((size_t)page * NV + c) * BS + (s0 - page * BS);
+#pragma unroll
+      for (int k = 0; k + 4 <= TR; k += 4) sta4(o, k, f32x4{v[k], v[k + 1], v[k + 2], v[k + 3]});
+    } else if (vt) {
+#pragma unroll
+      for (int k = 0; k < TR; ++k) {
+        const int sl = k < nr ? slots[r0 + k] : -1;
+        if (sl >= 0) sta(vt, ((size_t)(sl / BS) * NV + c) * BS + sl % BS, v[k]);
+      }
+    }
+    if (vc) {
+#pragma unroll
+      for (int k = 0; k < TR; ++k) {
+        const int sl = k < nr ? slots[r0 + k] : -1;
+        if (sl >= 0) sta(vc, (size_t)sl * NV + c, v[k]);
+      }
+    }
+  }
+}
+
 // The preparation where a row's entries do not meet beyond their rotation pair (2i, 2i + 1): no norm, no bias,
 // cos | sin from the table.  A thread takes four neighbouring entries -- two pairs -- at a time straight from
 // memory to memory (no LDS).  A workgroup takes TR rows; value column c of TR rows whose slots are TR aligned
@@ -215,34 +252,74 @@ __global__ void __launch_bounds__(256) attn_prep_pairs_kernel(const float* __res
       if (sl >= 0) sta4(kc, (size_t)sl * NK + (c - NQ), v);
     }
   }
-  if (NV == 0) return;
-  const int s0 = slots[r0];
-  bool run = TR > 1 && nr == TR && s0 >= 0 && s0 % TR == 0 && BS % TR == 0;    // then a page holds all TR
-  for (int k = 1; k < nr; ++k) run = run && slots[r0 + k] == s0 + k;
-  for (int c = tid; c < NV; c += 256) {
-    float v[TR];
+  write_values<TA, TR>(x, qs, r0, nr, NV, v_col, nullptr, slots, vc, vt, BS, tid);
+}
+
+// The preparation with rotation halves (i with i + rot / 2), biases and a norm per head behind the rotation, cos | sin from
+// the table:  D / 8 neighbouring lanes (a power of two) hold a head, each two groups of four entries -- rotated ones and
+// their partners, or eight neighbours behind the rotated part -- so the rotation needs no exchange, the norm a few
+// cross-lane sums, and every access is 16 bytes.
+template <typename TA, int TR>
+__global__ void __launch_bounds__(256) attn_prep_half_kernel(const float* __restrict__ x, int qs, int H, int G, int NV, int D,
+                                                             int v_col, const float* __restrict__ bias,
+                                                             const int* __restrict__ slots, TA* __restrict__ kc,
+                                                             TA* __restrict__ vc, TA* __restrict__ vt, int BS,
+                                                             TA* __restrict__ q_out, int rot, const float* __restrict__ cs,
+                                                             int norm, const float* __restrict__ q_w,
+                                                             const float* __restrict__ k_w, float eps, int T) {
+  const int r0 = blockIdx.x * TR, tid = threadIdx.x, half = rot >> 1, lph = D >> 3, units = H + G;
+  const int nr = min(TR, T - r0), n = units * lph;
+  for (int i = tid; i < nr * n; i += 256) {
+    const int rr = i / n, u = (i - rr * n) / lph, j = i & (lph - 1), r = r0 + rr;
+    const bool turn = 8 * j < rot;
+    const int a = turn ? 4 * j : 8 * j, b = turn ? a + half : a + 4;
+    const float* p = x + (size_t)r * qs + u * D;
+    f32x4 va = *reinterpret_cast<const f32x4*>(p + a), vb = *reinterpret_cast<const f32x4*>(p + b);
+    if (bias) {
 #pragma unroll
-    for (int k = 0; k < TR; ++k) v[k] = k < nr ? x[(size_t)(r0 + k) * qs + v_col + c] : 0.f;
-    if (vt && run) {
-      const int page = s0 / BS;
-      TA* o = vt + ((size_t)page * NV + c) * BS + (s0 - page * BS);
-#pragma unroll
-      for (int k = 0; k + 4 <= TR; k += 4) sta4(o, k, f32x4{v[k], v[k + 1], v[k + 2], v[k + 3]});
-    } else if (vt) {
-#pragma unroll
-      for (int k = 0; k < TR; ++k) {
-        const int sl = k < nr ? slots[r0 + k] : -1;
-        if (sl >= 0) sta(vt, ((size_t)(sl / BS) * NV + c) * BS + sl % BS, v[k]);
+      for (int k = 0; k < 4; ++k) {
+        va[k] += bias[u * D + a + k];
+        vb[k] += bias[u * D + b + k];
       }
     }
-    if (vc) {
+    if (turn) {
+      const float* c = cs + (size_t)r * rot + a;
+      const f32x4 co = *reinterpret_cast<const f32x4*>(c), si = *reinterpret_cast<const f32x4*>(c + half);
 #pragma unroll
-      for (int k = 0; k < TR; ++k) {
-        const int sl = k < nr ? slots[r0 + k] : -1;
-        if (sl >= 0) sta(vc, (size_t)sl * NV + c, v[k]);
+      for (int k = 0; k < 4; ++k) {
+        const float ua = va[k], ub = vb[k];
+        va[k] = ua * co[k] - ub * si[k];
+        vb[k] = ub * co[k] + ua * si[k];
+      }
+    }
+    float rn = 1.f;
+    if (norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) ss = fmaf(va[k], va[k], fmaf(vb[k], vb[k], ss));
+      for (int o = 1; o < lph; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      rn = 1.f / sqrtf(ss / (float)D + eps);
+    }
+    const float* w = u < H ? q_w : k_w;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      va[k] *= rn * (w ? w[a + k] : 1.f);
+      vb[k] *= rn * (w ? w[b + k] : 1.f);
+    }
+    if (u < H) {
+      const size_t o = ((size_t)r * H + u) * D;
+      sta4(q_out, o + a, va);
+      sta4(q_out, o + b, vb);
+    } else {
+      const int sl = slots[r];
+      if (sl >= 0) {
+        const size_t o = ((size_t)sl * G + u - H) * D;
+        sta4(kc, o + a, va);
+        sta4(kc, o + b, vb);
       }
     }
   }
+  write_values<TA, TR>(x, qs, r0, nr, NV, v_col, bias, slots, vc, vt, BS, tid);
 }
 
 // The visible keys of position `pos`: [a0, a1) and [lo, pos], walked as x in [0, nA + nB).
@@ -744,6 +821,31 @@ K8S_API int k8s_attn_prep_pairs(const float* x, int qs, int H, int G, int D, int
     else K8S_PP(float, 1);
   }
 #undef K8S_PP
+  return (int)hipGetLastError();
+}
+
+// D 8, 16, .. 512 (powers of two), qs a multiple of 4, rot a multiple of 8 with its table, x / q_out / kc / cs 16-byte
+// aligned (8 for bf16 outputs); norm 0 / 1 as in k8s_attn_prep
+K8S_API int k8s_attn_prep_half(const float* x, int qs, int H, int G, int D, int NV, int v_col, const float* bias,
+                               const int* slots, void* kc, void* vc, void* vt, int BS, void* q_out, int dt, int rot,
+                               const float* cs, int norm, const float* q_w, const float* k_w, float eps, int T,
+                               hipStream_t s) {
+  if (T <= 0) return 0;
+  if (H < 1 || G < 0 || D < 8 || D > 512 || (D & (D - 1)) || qs % 4 || rot < 0 || rot > D || rot % 8 || (rot && !cs) ||
+      NV < 0 || v_col < 0 || BS < 1 || (G > 0 && !kc) || (NV > 0 && !vc && !vt) || norm < 0 || norm > 1 ||
+      ((uintptr_t)x & 15) || ((uintptr_t)cs & 15))
+    return (int)hipErrorInvalidValue;
+#define K8S_PH(TA, TR)                                                                                                   \
+  hipLaunchKernelGGL((attn_prep_half_kernel<TA, TR>), dim3((T + TR - 1) / TR), dim3(256), 0, s, x, qs, H, G, NV, D, v_col, \
+                     bias, slots, (TA*)kc, (TA*)vc, (TA*)vt, BS, (TA*)q_out, rot, cs, norm, q_w, k_w, eps, T)
+  if (dt == 0) {
+    if (T > 1024) K8S_PH(uint16_t, 8);
+    else K8S_PH(uint16_t, 1);
+  } else {
+    if (T > 1024) K8S_PH(float, 8);
+    else K8S_PH(float, 1);
+  }
+#undef K8S_PH
   return (int)hipGetLastError();
 }
 

@@ -124,6 +124,7 @@ _SIGS = {
     "k8s_attn_prep": [P, I, P, I, I, I, I, P, P, P, P, P, I, P, I, I, P, P, F, I, F, F, P, P, I, P, I, F, I, P, F, I, P],
     "k8s_rope_table": [P, P, F, P, I, I, P],
     "k8s_attn_prep_pairs": [P, I, I, I, I, I, I, P, P, P, P, I, P, I, I, P, I, P],
+    "k8s_attn_prep_half": [P, I, I, I, I, I, I, P, P, P, P, P, I, P, I, I, P, I, P, P, F, I, P],
     "k8s_masked_attn_rows": [P, P, P, P, I, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, I, F, F, I, P, I, I],
     "k8s_masked_attn_mfma_ok": [I, I, I, I],
     "k8s_masked_attn_mfma": [P, P, P, P, I, P, I, P, P, I, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, P, I, I],

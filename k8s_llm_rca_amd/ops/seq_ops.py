@@ -628,7 +628,9 @@ def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor
         longest = max(b - a for a, b in zip(seg.row0_host[:-1], seg.row0_host[1:]))
         mfma = longest >= LIN_MFMA_ROWS and decay_mfma_ok(D, V, x.dtype, x.device) and x.stride(0) % 4 == 0
         if mfma:
-            cr = seg.chunk_ranges(LIN_CHUNK, LIN_CHUNK) if seg.n_seg * H * -(-V // 128) < LIN_FILL_GROUPS else None
+            ranges = max(1, LIN_GROUPS // (H * -(-V // 128)))      # as many as give the chip a workgroup per unit
+            rows = max(LIN_CHUNK, -(-T // (64 * ranges)) * 64)
+            cr = seg.chunk_ranges(rows, rows)                       # (None: no portion is longer than a range)
         else:
             cr = seg.chunk_ranges(SSM_CHUNK, 2 * SSM_CHUNK) if seg.n_seg * H * V * 8 < SEQ_FILL_LANES else None
         chunks, c0, cs, nch = None, None, None, 0
@@ -660,8 +662,8 @@ def decay_attention(x: torch.Tensor, H: int, D: int, V: int, decay: torch.Tensor
 
 
 LIN_MFMA_ROWS = 17      # rows of a step's longest portion from which the matrix-core form runs
-LIN_CHUNK = 128         # rows per range where ranges of a portion run in parallel
-LIN_FILL_GROUPS = 128   # workgroups (segments x heads x 128 value columns) from which whole portions fill the chip
+LIN_CHUNK = 128         # rows at least per range where ranges of a portion run in parallel
+LIN_GROUPS = 256        # workgroups (ranges x heads x 128 value columns) a step is cut into
 
 
 def decay_mfma_ok(D: int, V: int, dtype, device) -> bool:
@@ -881,6 +883,14 @@ def attn_prep(qkv: torch.Tensor, bias: Optional[torch.Tensor], H: int, G: int, D
             check(lib().k8s_attn_prep_pairs(ptr(qkv), qkv.stride(0), HQ, GK, D, NV, v_col, ptr(slots), ptr(kc), ptr(vc),
                                             ptr(vt), BS, ptr(q_out), _dt(out_dtype), int(rot_dims), ptr(rope_cs), T,
                                             stream_ptr(qkv)), "attn_prep_pairs")
+            return q_out
+        if (mode < 2 and v_other is None and v_keep is None and not tq_every and 8 <= D <= 512 and D & (D - 1) == 0
+                and qkv.stride(0) % 4 == 0 and qkv.data_ptr() % 16 == 0 and rot_dims % 8 == 0
+                and (rot_dims == 0 or (rope is not None and not rope.pairs and rope_cs is not None))):
+            # a head's entries meet in its rotation and its norm alone: a few lanes per head, no LDS
+            check(lib().k8s_attn_prep_half(ptr(qkv), qkv.stride(0), HQ, GK, D, NV, v_col, ptr(bias), ptr(slots), ptr(kc),
+                                           ptr(vc), ptr(vt), BS, ptr(q_out), _dt(out_dtype), int(rot_dims), ptr(rope_cs),
+                                           mode, ptr(q_w), ptr(k_w), float(eps), T, stream_ptr(qkv)), "attn_prep_half")
             return q_out
         check(lib().k8s_attn_prep(ptr(qkv), qkv.stride(0), ptr(bias), HQ, GK, D, NV, ptr(positions), ptr(slots),
                                   ptr(kc), ptr(vc), ptr(vt), BS, ptr(q_out), _dt(out_dtype), mode, ptr(q_w),

@@ -520,8 +520,8 @@ def test_decaying_memory_across_portions_and_slots(backend, H, D, V, silu, monke
     want, Sw = decay_reference(x[:, :-4], H, D, V, decay, torch.zeros(H, D, V, dtype=DT), silu, dt)
     xd = x.to(dev).to(dt)
     tol = torch.float32 if dt == torch.float32 else torch.bfloat16
-    for fill, cuts in [(128, (T,)), (0, (T,)), (128, (64, 1, 1, 63, 200, 1)), (0, (130, 2, 17, 100)), (128, (2, 3, 1, 20, 304))]:
-        monkeypatch.setattr(S, "LIN_FILL_GROUPS", fill)
+    for fill, cuts in [(1 << 20, (T,)), (0, (T,)), (256, (64, 1, 1, 63, 200, 1)), (0, (130, 2, 17, 100)), (1 << 20, (2, 3, 1, 20, 304))]:
+        monkeypatch.setattr(S, "LIN_GROUPS", fill)
         state = torch.full((3, H, D, V), float("nan"), device=dev)
         got = in_portions(lambda a, e: S.decay_attention(xd[a:e, :-4], H, D, V, f32(decay, dev), state,
                                                          seg_meta([e - a], [a], [1], dev), silu=silu), T, cuts)
@@ -532,11 +532,11 @@ def test_decaying_memory_across_portions_and_slots(backend, H, D, V, silu, monke
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
-@pytest.mark.parametrize("D,V,fill", [(16, 24, 128), (64, 64, 128), (64, 64, 0), (128, 32, 128)])
+@pytest.mark.parametrize("D,V,fill", [(16, 24, 256), (64, 64, 1 << 20), (64, 64, 0), (128, 32, 1 << 20)])
 def test_sequences_in_one_step_keep_their_own_memory(backend, D, V, fill, monkeypatch):
     """A long portion beside a short one and a single token, slots not in segment order: each gets what it gets alone."""
     dev, dt = backend
-    monkeypatch.setattr(S, "LIN_FILL_GROUPS", fill)
+    monkeypatch.setattr(S, "LIN_GROUPS", fill)
     H, lens, pos0, slots = 3, [200, 3, 1, 65], [0, 5, 9, 64], [2, 0, 3, 1]
     T = sum(lens)
     x = b16(rnd(T, H * (2 * D + V), seed=1)).to(dev).to(dt)
