@@ -193,7 +193,7 @@ def _stack(heads: int, kv_heads: int, dim: int, q_rank: int, kv_rank: int, rot_d
 
 
 PRESETS: Dict[str, FikeraxConfig] = {
-    "tiny-fikerax": FikeraxConfig("tiny-fikerax", 8192, 256, _stack(4, 2, 64, 96, 64, 32, 128, 512), embed_scale=16.0,
+    "tiny-fikerax": FikeraxConfig("tiny-fikerax", 8192, 384, _stack(6, 3, 64, 80, 96, 32, 160, 640), embed_scale=18.0,
                                   loop=(1, 4, 2)),
     # sizes of a ~1B-class decoder's layers (benchmarks; random weights): 1 + 3 x 3 + 1 layer runs
     "fikerax-1b": FikeraxConfig("fikerax-1b", 32768, 2048, _stack(16, 2, 128, 768, 256, 64, 1024, 8192),

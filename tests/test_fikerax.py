@@ -245,7 +245,7 @@ def test_residual_reads_the_embedding_output_again(backend, W, streams):
 
 
 @pytest.mark.parametrize("dims,base,sc", [
-    (64, 50000.0, {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 300}), (6, 300.0, STRETCH), (2, 10.0, STRETCH),
+    (64, 20000.0, {"factor": 6.0, "low": 1.5, "high": 5.0, "original": 300}), (6, 300.0, STRETCH), (2, 10.0, STRETCH),
     (32, 5000.0, {"factor": 2.5, "low": 0.5, "high": 20.0, "original": 1000}),
     (16, 1e6, {"factor": 1.0, "low": 1.0, "high": 2.0, "original": 64}), (8, 77.0, None)])
 def test_stretched_frequencies(dims, base, sc):
@@ -394,7 +394,7 @@ def test_latent_attention_with_a_shared_key_part(backend, H, R, P, window, sink)
 
 
 @pytest.mark.parametrize("backend", MFMA_BACKEND)
-@pytest.mark.parametrize("H,R,P,window", [(8, 64, 32, 72), (16, 256, 64, 200), (3, 32, 32, 1), (1, 128, 0, 33), (24, 96, 32, 64),
+@pytest.mark.parametrize("H,R,P,window", [(6, 64, 32, 75), (16, 256, 64, 200), (3, 32, 32, 1), (1, 128, 0, 33), (24, 96, 32, 64),
                                           (5, 192, 64, 0), (40, 64, 64, 130), (7, 512, 32, 300), (2, 384, 64, 96)])
 def test_latent_attention_on_the_matrix_cores(backend, H, R, P, window):
     """Prompt portions and decoding rows (their keys split over partitions) against the plain softmax; two sequences of
@@ -474,7 +474,7 @@ def masked_case(dev, dt, H, G, D, V, n, BS, seed, sharp=None):
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("aim", ["edge_in", "edge_out", "page_first", "future"])
-@pytest.mark.parametrize("H,G,D,V,window", [(6, 3, 8, 10, 70), (4, 2, 64, 64, 96), (4, 2, 128, 64, 33), (2, 1, 64, 64, 1)])
+@pytest.mark.parametrize("H,G,D,V,window", [(6, 3, 8, 10, 70), (6, 2, 64, 64, 90), (4, 2, 128, 64, 33), (2, 1, 64, 64, 1)])
 def test_one_key_stands_out_in_the_windowed_attention(backend, aim, H, G, D, V, window):
     dev, dt = backend
     n, BS, i = 302, 32, 300
@@ -678,8 +678,8 @@ def test_sharp_scores_over_page_borders(backend):
         assert agrees(got, want, backend[1], mult=2.0 if backend[1] == torch.float32 else 3.5), (cuts, row_errs(got, want).max())
 
 
-BIG = [(lig(heads=2, dim=64, vdim=64), 0), (att(heads=4, kv_heads=2, dim=64, vdim=64, rot=64, scale=0.3, window=96), 64),
-       (lat(heads=4, dim=32, rot=16, vdim=32, q_rank=48, kv_rank=64, window=72), 64)]
+BIG = [(lig(heads=2, dim=64, vdim=64), 0), (att(heads=6, kv_heads=2, dim=64, vdim=64, rot=48, scale=0.3, window=90), 64),
+       (lat(heads=5, dim=24, rot=20, vdim=40, q_rank=48, kv_rank=96, window=75), 56)]
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
